@@ -30,7 +30,7 @@
 // ------------------------------------------------------------------ prefill
 // grid (ceil(max_q_len / 64), H, num_seqs), 256 threads: wave w takes the 16
 // queries q0 = 64*blockIdx.x + 16*w of the sequence.
-template <int NT, bool BIAS>
+template <int NT, int MODE>
 __global__ __launch_bounds__(256) void attention_prefill_kernel(
     uint16_t* __restrict__ out, const uint16_t* __restrict__ q,
     const uint16_t* __restrict__ kpool, const uint16_t* __restrict__ vpool,
@@ -65,7 +65,8 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(
   for (int dt = 0; dt < NT; ++dt) st.o[dt] = floatx4{0.f, 0.f, 0.f, 0.f};
   st.m = -INFINITY;
   st.l = 0.f;
-  st.bias = BIAS ? ex.slopes[h] / scale : 0.f;
+  st.bias = MODE == ATTN_SLOPES ? ex.slopes[h] / scale : 0.f;
+  if (MODE == ATTN_SHAPED) st.sh = attn_shape_of(ex, h, scale);
   st.pos = pos;
 
   const int last_pos = start + min(q0 + 15, q_len - 1);
@@ -76,8 +77,8 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(
   const bool full_tile = q0 + 15 < q_len;
   const int clear_lo = attn_first(last_pos, window, ex.chunk);
   const int clear_hi = full_tile ? first_pos : -1;
-  attend_range<NT, true, BIAS>(st, qf, kpool, vpool, pt, max_blocks, num_pages, KVH, kvh, tile_lo & ~31,
-                   (last_pos & ~31) + 32, lo, hi, clear_lo, clear_hi, scale * 1.4426950408889634f,
+  attend_range<NT, true, MODE>(st, qf, kpool, vpool, pt, max_blocks, num_pages, KVH, kvh, tile_lo & ~31,
+                   (last_pos & ~31) + 32, lo, hi, clear_lo, clear_hi, MODE == ATTN_SHAPED ? 1.f : scale * 1.4426950408889634f,
                    lr, lg);
   float l = st.l;
   l = xor32_sum(xor16_sum(l));
@@ -104,7 +105,7 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(
 // With a single slice in the grid the result is written directly.
 #define DECODE_MIN_CHUNK 64
 
-template <int NT, bool BIAS>
+template <int NT, int MODE>
 __global__ __launch_bounds__(64) void attention_decode_kernel(
     uint16_t* __restrict__ out, float* __restrict__ ws_o, float* __restrict__ ws_ml,
     const uint16_t* __restrict__ q,
@@ -150,11 +151,12 @@ __global__ __launch_bounds__(64) void attention_decode_kernel(
   for (int dt = 0; dt < NT; ++dt) st.o[dt] = floatx4{0.f, 0.f, 0.f, 0.f};
   st.m = -INFINITY;
   st.l = 0.f;
-  st.bias = BIAS ? ex.slopes[h] / scale : 0.f;
+  st.bias = MODE == ATTN_SLOPES ? ex.slopes[h] / scale : 0.f;
+  if (MODE == ATTN_SHAPED) st.sh = attn_shape_of(ex, h, scale);
   st.pos = n_keys - 1;
   const int hi = n_keys - 1;
-  attend_range<NT, false, BIAS>(st, qf, kpool, vpool, pt, max_blocks, num_pages, KVH, kvh, kb_begin,
-                   (kb_end + 31) & ~31, first, hi, first, hi, scale * 1.4426950408889634f, lr, lg);
+  attend_range<NT, false, MODE>(st, qf, kpool, vpool, pt, max_blocks, num_pages, KVH, kvh, kb_begin,
+                   (kb_end + 31) & ~31, first, hi, first, hi, MODE == ATTN_SHAPED ? 1.f : scale * 1.4426950408889634f, lr, lg);
   float l = st.l;
   l = xor32_sum(xor16_sum(l));
   if (nsplit == 1) {                      // nothing to merge
@@ -310,8 +312,13 @@ extern "C" int he_attention_decode_bf16(void* out, const void* q, const void* kp
                                         int max_keys, void* workspace_f32,
                                         int64_t workspace_floats, int chunk, const void* sinks,
                                         int sinks_dtype, const void* gate, int64_t gate_stride,
-                                        const void* slopes_f32, void* stream) {
-  const AttnExtras ex = {sinks, sinks_dtype, (const uint16_t*)gate, gate_stride, chunk, (const float*)slopes_f32};
+                                        const void* slopes_f32, const void* table_f32, int table_len,
+                                        float cap, void* stream) {
+  const AttnExtras ex = {sinks, sinks_dtype, (const uint16_t*)gate, gate_stride, chunk, (const float*)slopes_f32,
+                         (const float*)table_f32, table_len, cap};
+  HE_REQUIRE(slopes_f32 == nullptr || (table_f32 == nullptr && !(cap > 0.f)),
+             "he_attention_decode_bf16: slopes go with neither a cap nor a distance table");
+  HE_REQUIRE(table_f32 == nullptr || table_len > 0, "he_attention_decode_bf16: an empty distance table");
   HE_REQUIRE(rows >= 0 && H > 0 && KVH > 0 && hd > 0 && max_keys > 0,
              "he_attention_decode_bf16: bad sizes");
   HE_REQUIRE(scale > 0.f, "he_attention_decode_bf16: the score scale must be positive");
@@ -340,10 +347,10 @@ extern "C" int he_attention_decode_bf16(void* out, const void* q, const void* kp
   (uint16_t*)out, ws_o, ws_ml, (const uint16_t*)q, (const uint16_t*)kpool, (const uint16_t*)vpool,     \
       (const int32_t*)positions, (const int32_t*)row_seq, (const int32_t*)seq_slot,                    \
       (const int32_t*)page_table, max_blocks, num_pages, H, KVH, head_tiles, window, scale, ex
-  if (ex.slopes != nullptr) {
-    ATTN_SWITCH(hd / 16, (attention_decode_kernel<NT, true><<<grid, 64, 0, s>>>(DECODE_ARGS)));
-  } else {
-    ATTN_SWITCH(hd / 16, (attention_decode_kernel<NT, false><<<grid, 64, 0, s>>>(DECODE_ARGS)));
+  switch (attn_mode(ex)) {
+    case ATTN_SLOPES: ATTN_SWITCH(hd / 16, (attention_decode_kernel<NT, ATTN_SLOPES><<<grid, 64, 0, s>>>(DECODE_ARGS))); break;
+    case ATTN_SHAPED: ATTN_SWITCH(hd / 16, (attention_decode_kernel<NT, ATTN_SHAPED><<<grid, 64, 0, s>>>(DECODE_ARGS))); break;
+    default: ATTN_SWITCH(hd / 16, (attention_decode_kernel<NT, ATTN_RAW><<<grid, 64, 0, s>>>(DECODE_ARGS)));
   }
 #undef DECODE_ARGS
   int rc = he_check_launch("he_attention_decode_bf16");
@@ -450,8 +457,14 @@ extern "C" int he_attention_prefill_bf16(void* out, const void* q, const void* k
                                          int parts, void* workspace_f32, int64_t workspace_floats,
                                          int chunk, const void* sinks, int sinks_dtype,
                                          const void* gate, int64_t gate_stride, const void* slopes_f32,
-                                         void* stream) {
-  const AttnExtras ex = {sinks, sinks_dtype, (const uint16_t*)gate, gate_stride, chunk, (const float*)slopes_f32};
+                                         const void* table_f32, int table_len, float cap, void* stream) {
+  const AttnExtras ex = {sinks, sinks_dtype, (const uint16_t*)gate, gate_stride, chunk, (const float*)slopes_f32,
+                         (const float*)table_f32, table_len, cap};
+  HE_REQUIRE(slopes_f32 == nullptr || (table_f32 == nullptr && !(cap > 0.f)),
+             "he_attention_prefill_bf16: slopes go with neither a cap nor a distance table");
+  HE_REQUIRE(table_f32 == nullptr || table_len > 0, "he_attention_prefill_bf16: an empty distance table");
+  HE_REQUIRE(kernel < 2 || table_f32 == nullptr || table_len <= HE_ATTN_TABLE_LDS,
+             "he_attention_prefill_bf16: kernel 2 takes distance tables of up to %d entries, not %d", HE_ATTN_TABLE_LDS, table_len);
   HE_REQUIRE(num_seqs >= 0 && max_q_len >= 0 && H > 0 && KVH > 0 && hd > 0 && total_rows >= 0,
              "he_attention_prefill_bf16: bad sizes");
   HE_REQUIRE(kernel >= 0 && kernel <= 2,
@@ -470,7 +483,7 @@ extern "C" int he_attention_prefill_bf16(void* out, const void* q, const void* k
              "he_attention_prefill_bf16: buffers must be 16-byte aligned");
   if (num_seqs == 0 || max_q_len == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  if (kernel == 0) kernel = hd > 128 ? 1 : 2;
+  if (kernel == 0) kernel = hd > 128 || (table_f32 != nullptr && table_len > HE_ATTN_TABLE_LDS) ? 1 : 2;
   if (parts < 1) parts = 1;
   HE_REQUIRE(parts == 1 || kernel == 2,
              "he_attention_prefill_bf16: keys in %d parts are for kernel 2 (head sizes up to 128)", parts);
@@ -494,10 +507,10 @@ extern "C" int he_attention_prefill_bf16(void* out, const void* q, const void* k
   (uint16_t*)out, (const uint16_t*)q, (const uint16_t*)kpool, (const uint16_t*)vpool,                  \
       (const int32_t*)cu_seqlens, (const int32_t*)seq_slot, (const int32_t*)seq_start,                 \
       (const int32_t*)page_table, max_blocks, num_pages, H, KVH, window, scale, ex
-  if (ex.slopes != nullptr) {
-    ATTN_SWITCH(hd / 16, (attention_prefill_kernel<NT, true><<<grid, 256, 0, s>>>(PREFILL_ARGS)));
-  } else {
-    ATTN_SWITCH(hd / 16, (attention_prefill_kernel<NT, false><<<grid, 256, 0, s>>>(PREFILL_ARGS)));
+  switch (attn_mode(ex)) {
+    case ATTN_SLOPES: ATTN_SWITCH(hd / 16, (attention_prefill_kernel<NT, ATTN_SLOPES><<<grid, 256, 0, s>>>(PREFILL_ARGS))); break;
+    case ATTN_SHAPED: ATTN_SWITCH(hd / 16, (attention_prefill_kernel<NT, ATTN_SHAPED><<<grid, 256, 0, s>>>(PREFILL_ARGS))); break;
+    default: ATTN_SWITCH(hd / 16, (attention_prefill_kernel<NT, ATTN_RAW><<<grid, 256, 0, s>>>(PREFILL_ARGS)));
   }
 #undef PREFILL_ARGS
   return he_check_launch("he_attention_prefill_bf16");

@@ -11,7 +11,8 @@
 // s_j = (q . k_j) * scale for j in [first, p], out = sum_j softmax(s)_j v_j,
 // kv head = h / (H / KVH)   (reference: kernels/attention.cu:155-316, :664-773, :60).
 // sinks (one number a head, or null): the softmax's denominator also holds exp(sink_h), which has no
-// key and no value; it joins last, after the pages. gate (one number a row and head, or null): the
+// key and no value; it joins last, after the pages. A score may fall with the distance by a slope a head, or be
+// capped and then shifted by a table a head over the distance (ap_shape). gate (one number a row and head, or null): the
 // head's output is multiplied by sigmoid(gate) before it is stored.
 //
 // Three launches keep that order and give the same bits: one wavefront per (query, head) that walks
@@ -26,7 +27,7 @@
 #include "cache_layout.h"
 #include "hector_kernels.h"
 
-#define AP_MAX_PER_LANE 8
+#define AP_MAX_PER_LANE 16
 
 // the first key the query at position p sees
 __device__ __forceinline__ int ap_first(int p, int window, int chunk) {
@@ -35,7 +36,7 @@ __device__ __forceinline__ int ap_first(int p, int window, int chunk) {
   return first;
 }
 
-// NPL: head elements a lane holds (head_dim / 64 rounded up to 1, 2, 4 or 8)
+// NPL: head elements a lane holds (head_dim / 64 rounded up to 1, 2, 4, 8 or 16)
 template <int NPL>
 struct ApState {
   float m, l;
@@ -75,6 +76,19 @@ __device__ __forceinline__ void ap_update(ApState<NPL>& st, float s, const float
   st.m = m_new;
 }
 
+// What shapes a score beyond q . k * scale: a slope over the distance, or a cap and a table over the distance (of this head).
+struct ApShape {
+  float slope, cap;
+  const float* table;    // the head's entries, or null
+  int last;              // the table's last index
+};
+// the score of a key `back` positions before the query (negative: a key the caller leaves out)
+__device__ __forceinline__ float ap_shape(const ApShape& sh, float s, int back) {
+  if (sh.cap > 0.f) s = sh.cap * tanhf(s / sh.cap);
+  if (sh.table != nullptr) return s + sh.table[min(max(back, 0), sh.last)];
+  return fmaf(sh.slope, (float)-back, s);
+}
+
 #define AP_GROUP 4
 // The key and value elements of this lane for the AP_GROUP keys from j0 on (positions beyond j_hi
 // read key j_hi again: no load stands behind a condition, so the compiler counts what is in flight).
@@ -101,8 +115,8 @@ __device__ __forceinline__ void ap_fetch(float (&kv)[AP_GROUP][NPL], float (&vv)
 template <typename T, int NPL>
 __device__ __forceinline__ void ap_page(ApState<NPL>& st, const float (&qv)[NPL], const T* kpool,
                                         const T* vpool, int page, int num_pages, int KVH, int kvh, int hd,
-                                        int j_lo, int j_hi, float scale, int lane, int npl, float slope = 0.f,
-                                        int p = 0) {
+                                        int j_lo, int j_hi, float scale, int lane, int npl, const ApShape& sh,
+                                        int p) {
   st.m = -INFINITY;
   st.l = 0.f;
 #pragma unroll
@@ -123,14 +137,14 @@ __device__ __forceinline__ void ap_page(ApState<NPL>& st, const float (&qv)[NPL]
     float sc[AP_GROUP];
 #pragma unroll
     for (int g = 0; g < AP_GROUP; ++g)
-      sc[g] = fmaf(slope, (float)(j0 + g - p), ap_score<NPL>(qv, ka[g], scale, lane, npl, hd));
+      sc[g] = ap_shape(sh, ap_score<NPL>(qv, ka[g], scale, lane, npl, hd), p - (j0 + g));
 #pragma unroll
     for (int g = 0; g < AP_GROUP; ++g)
       if (j0 + g <= j_hi) ap_update<NPL>(st, sc[g], va[g], lane, npl, hd);
     ap_fetch<T, NPL>(ka, va, kpage, vpage, j0 + 2 * AP_GROUP, j_hi, KS, NT, lane, npl, hd);
 #pragma unroll
     for (int g = 0; g < AP_GROUP; ++g)
-      sc[g] = fmaf(slope, (float)(j0 + AP_GROUP + g - p), ap_score<NPL>(qv, kb[g], scale, lane, npl, hd));
+      sc[g] = ap_shape(sh, ap_score<NPL>(qv, kb[g], scale, lane, npl, hd), p - (j0 + AP_GROUP + g));
 #pragma unroll
     for (int g = 0; g < AP_GROUP; ++g)
       if (j0 + AP_GROUP + g <= j_hi) ap_update<NPL>(st, sc[g], vb[g], lane, npl, hd);
@@ -157,7 +171,14 @@ struct ApExtras {
   const void* gate;      // gate[row * gate_stride + h] in the activation dtype, or null
   int64_t gate_stride;
   const float* slopes;   // [H] or null: the score of key j for the query at p loses slopes[h] * (p - j)
+  const float* table;    // [H][table_len] or null: the score gains table[h][min(p - j, table_len - 1)]
+  int table_len;
+  float cap;             // > 0: a score s becomes cap * tanh(s / cap) first
 };
+__device__ __forceinline__ ApShape ap_shape_of(const ApExtras& ex, int h) {
+  return ApShape{ex.slopes ? ex.slopes[h] : 0.f, ex.cap, ex.table ? ex.table + (int64_t)h * ex.table_len : nullptr,
+                 ex.table_len - 1};
+}
 template <typename T, int NPL>
 __device__ __forceinline__ float ap_finish(ApState<NPL>& total, const ApExtras& ex, int64_t row, int h) {
   if (ex.sinks != nullptr) {
@@ -202,7 +223,7 @@ __global__ __launch_bounds__(256) void attention_plain_kernel(
   const int p = positions[row];
   const int slot = seq_slot[seq];
   const int kvh = h / (H / KVH);
-  const float slope = ex.slopes ? ex.slopes[h] : 0.f;
+  const ApShape sh = ap_shape_of(ex, h);
   const int first = ap_first(p, window, chunk);
   const int32_t* pt = page_table + (int64_t)slot * max_blocks;
   const int c_first = first >> HE_PAGE_SHIFT, c_last = p >> HE_PAGE_SHIFT;
@@ -219,7 +240,7 @@ __global__ __launch_bounds__(256) void attention_plain_kernel(
   if (split) {
     const int c = c_first + blockIdx.z;
     ap_page<T, NPL>(st, qv, kpool, vpool, pt[c], num_pages, KVH, kvh, hd, max(first, c << HE_PAGE_SHIFT),
-               min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, slope, p);
+               min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, sh, p);
     float* w = ws + ((row * H + h) * (int64_t)gridDim.z + blockIdx.z) * (hd + 2);
 #pragma unroll
     for (int i = 0; i < NPL; ++i) {
@@ -236,7 +257,7 @@ __global__ __launch_bounds__(256) void attention_plain_kernel(
   for (int i = 0; i < NPL; ++i) total.acc[i] = 0.f;
   for (int c = c_first; c <= c_last; ++c) {
     ap_page<T, NPL>(st, qv, kpool, vpool, pt[c], num_pages, KVH, kvh, hd, max(first, c << HE_PAGE_SHIFT),
-               min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, slope, p);
+               min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, sh, p);
     ap_join(total, st);
   }
   const float gf = ap_finish<T, NPL>(total, ex, row, h);
@@ -267,7 +288,7 @@ __global__ __launch_bounds__(256) void attention_plain_rows_kernel(
   const int npl = (hd + HE_WAVE - 1) / HE_WAVE;
   const int kvh = h / (H / KVH);
   const int n_rows = (int)min((int64_t)AP_ROWS, rows - row0);
-  const float slope = ex.slopes ? ex.slopes[h] : 0.f;
+  const ApShape sh = ap_shape_of(ex, h);
   const int seq0 = row_seq[row0], p0 = positions[row0];
   bool together = n_rows == AP_ROWS && seq0 >= 0;
   for (int r = 1; r < n_rows; ++r) together = together && row_seq[row0 + r] == seq0 && positions[row0 + r] == p0 + r;
@@ -306,7 +327,7 @@ __global__ __launch_bounds__(256) void attention_plain_rows_kernel(
         load_q(qv, row);
         for (int c = first >> HE_PAGE_SHIFT; c <= (p >> HE_PAGE_SHIFT); ++c) {
           ap_page<T, NPL>(st, qv, kpool, vpool, pt[c], num_pages, KVH, kvh, hd, max(first, c << HE_PAGE_SHIFT),
-                          min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, slope, p);
+                          min(p, (c << HE_PAGE_SHIFT) + HE_PAGE_TOKENS - 1), scale, lane, npl, sh, p);
           ap_join(total, st);
         }
       }
@@ -354,7 +375,7 @@ __global__ __launch_bounds__(256) void attention_plain_rows_kernel(
         for (int g = 0; g < AP_GROUP; ++g)
 #pragma unroll
           for (int r = 0; r < AP_ROWS; ++r)
-            sc[g][r] = fmaf(slope, (float)(j0 + g - p0 - r), ap_score<NPL>(qv[r], ka[g], scale, lane, npl, hd));
+            sc[g][r] = ap_shape(sh, ap_score<NPL>(qv[r], ka[g], scale, lane, npl, hd), p0 + r - (j0 + g));
 #pragma unroll
         for (int g = 0; g < AP_GROUP; ++g) {
           const int j = j0 + g;
@@ -367,7 +388,7 @@ __global__ __launch_bounds__(256) void attention_plain_rows_kernel(
         for (int g = 0; g < AP_GROUP; ++g)
 #pragma unroll
           for (int r = 0; r < AP_ROWS; ++r)
-            sc[g][r] = fmaf(slope, (float)(j0 + AP_GROUP + g - p0 - r), ap_score<NPL>(qv[r], kb[g], scale, lane, npl, hd));
+            sc[g][r] = ap_shape(sh, ap_score<NPL>(qv[r], kb[g], scale, lane, npl, hd), p0 + r - (j0 + AP_GROUP + g));
 #pragma unroll
         for (int g = 0; g < AP_GROUP; ++g) {
           const int j = j0 + AP_GROUP + g;
@@ -474,7 +495,8 @@ extern "C" int he_attention_plain(void* out, const void* q, const void* kpool, c
                                   int H, int KVH, int hd, int window, int chunk, float scale,
                                   const void* sinks, int sinks_dtype, const void* gate,
                                   int64_t gate_stride, int dtype, int most_keys, void* workspace_f32,
-                                  int64_t workspace_floats, const void* slopes_f32, void* stream) {
+                                  int64_t workspace_floats, const void* slopes_f32, const void* table_f32,
+                                  int table_len, float cap, void* stream) {
   HE_REQUIRE(rows >= 0 && H > 0 && KVH > 0 && hd > 0, "he_attention_plain: bad sizes");
   HE_REQUIRE(H % KVH == 0, "he_attention_plain: heads %d not a multiple of kv heads %d", H, KVH);
   HE_REQUIRE(hd <= AP_MAX_PER_LANE * HE_WAVE, "he_attention_plain: head_dim %d above %d", hd,
@@ -482,8 +504,10 @@ extern "C" int he_attention_plain(void* out, const void* q, const void* kpool, c
   HE_REQUIRE(dtype == HE_BF16 || dtype == HE_F32, "he_attention_plain: unknown dtype %d", dtype);
   HE_REQUIRE(sinks == nullptr || sinks_dtype == HE_BF16 || sinks_dtype == HE_F32,
              "he_attention_plain: unknown dtype %d of the sinks", sinks_dtype);
+  HE_REQUIRE(slopes_f32 == nullptr || table_f32 == nullptr, "he_attention_plain: slopes and a distance table exclude each other");
+  HE_REQUIRE(table_f32 == nullptr || table_len > 0, "he_attention_plain: an empty distance table");
   if (rows == 0) return 0;
-  const ApExtras ex = {sinks, sinks_dtype, gate, gate_stride, (const float*)slopes_f32};
+  const ApExtras ex = {sinks, sinks_dtype, gate, gate_stride, (const float*)slopes_f32, (const float*)table_f32, table_len, cap};
   // page by page in parallel when the caller brought room for it (the same bits either way)
   const int64_t need = he_attention_plain_workspace_floats(rows, H, hd, most_keys, window, chunk);
   const bool split = need > 0 && workspace_f32 != nullptr && workspace_floats >= need;
@@ -500,18 +524,20 @@ extern "C" int he_attention_plain(void* out, const void* q, const void* kpool, c
 #define AP_JOIN(T, NPL)                                                                        \
   attention_plain_join_kernel<T, NPL><<<dim3(rows, (H + 3) / 4), 256, 0, s>>>(                 \
       (T*)out, ws, (const int32_t*)positions, (const int32_t*)row_seq, H, hd, window, chunk, pages, ex)
-  const int npl = (hd + HE_WAVE - 1) / HE_WAVE;   // elements a lane holds: 1, 2, up to 4, up to 8
+  const int npl = (hd + HE_WAVE - 1) / HE_WAVE;   // elements a lane holds: 1, 2, up to 4, up to 8, up to 16
 #define AP_BY_SIZE(WHAT)                                  \
   if (dtype == HE_BF16) {                                 \
     if (npl <= 1) WHAT(bf16_t, 1);                        \
     else if (npl <= 2) WHAT(bf16_t, 2);                   \
     else if (npl <= 4) WHAT(bf16_t, 4);                   \
-    else WHAT(bf16_t, 8);                                 \
+    else if (npl <= 8) WHAT(bf16_t, 8);                   \
+    else WHAT(bf16_t, 16);                                \
   } else {                                                \
     if (npl <= 1) WHAT(float, 1);                         \
     else if (npl <= 2) WHAT(float, 2);                    \
     else if (npl <= 4) WHAT(float, 4);                    \
-    else WHAT(float, 8);                                  \
+    else if (npl <= 8) WHAT(float, 8);                    \
+    else WHAT(float, 16);                                 \
   }
 #define AP_ROWS_LAUNCH(T, NPL)                                                                          \
   attention_plain_rows_kernel<T, NPL><<<dim3((rows + AP_ROWS - 1) / AP_ROWS, (H + 3) / 4), 256, 0, s>>>(   \

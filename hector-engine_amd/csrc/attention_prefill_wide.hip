@@ -50,6 +50,7 @@
 // fifths of what the matrix cores give at that clock; at 2048 tokens the launch is as long
 // as its longest wavefront (33 epochs of about 2650 cycles, 1024 of them products).
 #include "attention_tiles.h"
+#include "hector_kernels.h"
 
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16;
 typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
@@ -57,6 +58,7 @@ typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
 #define PW_WAVES 4
 #define PW_QUERIES (32 * PW_WAVES)
 #define PW_SLACK 16.0f
+#define PW_LOG2E 1.4426950408889634f
 
 template <int NT>
 struct Pw {
@@ -74,7 +76,8 @@ struct WideTile {
   floatx16 o[Pw<NT>::DT];    // O^T[32dt + 8a + 4g + r][query], i = 4a + r, unnormalised
   float m, l;                // reference point of the lane's query; this lane's share of the sum
   int lo, hi;                // keys the lane's query sees
-  float bias;                // BIAS kernels: the raw score of key j gains bias * (j - hi) (a distance slope over the scale)
+  float bias;                // ATTN_SLOPES: the raw score of key j gains bias * (j - hi) (a distance slope over the scale)
+  AttnShape sh;              // ATTN_SHAPED: its table lies in LDS, times log2(e) (an entry 0 where there is none)
 };
 
 // position of score i of a lane of half g inside its step of 32 keys
@@ -138,10 +141,10 @@ __device__ __forceinline__ void pw_epoch_end() {
 
 // What the score product of the step from key_base on starts from: zeros, or, with a distance slope, the slope's
 // share of every score, bias * (key - pos): the product adds q . k on top of it, so the softmax sees the sum.
-template <bool BIAS>
+template <int MODE>
 __device__ __forceinline__ floatx16 pw_score_start(float bias, int pos, int key_base, int g) {
   floatx16 s;
-  if (BIAS) {
+  if (MODE == ATTN_SLOPES) {
     const float base = bias * (float)(key_base + 8 * g - pos);
 #pragma unroll
     for (int i = 0; i < 16; ++i) s[i] = __builtin_fmaf(bias, (float)pw_key_of(i, 0), base);
@@ -180,11 +183,17 @@ __device__ __forceinline__ void pw_values(floatx16 (&o)[Pw<NT>::DT], const uint4
   }
 }
 
+// ATTN_SHAPED: raw score i of a step from key_base on through the cap and the table (base-2 domain).
+template <int NT>
+__device__ __forceinline__ float pw_shaped(const WideTile<NT>& t, float s, int i, int key_base, int g) {
+  return attn_cap(t.sh, s) + t.sh.table[min(max(t.hi - key_base - pw_key_of(i, g), 0), t.sh.last)];
+}
+
 // Softmax of one step of 32 keys from key_base on. Leaves P^T in p; the factor for the
 // accumulators in alpha when the reference point moved (the return value, the same in all
 // lanes). m and l are updated; the caller rescales o, after the value products of earlier
 // steps that are still under way.
-template <int NT>
+template <int NT, int MODE>
 __device__ __forceinline__ bool pw_softmax(WideTile<NT>& t, const floatx16& s, int key_base, int g,
                                            float scale_log2, bf16x8 (&p)[2], float& alpha) {
   float v[16];
@@ -192,7 +201,8 @@ __device__ __forceinline__ bool pw_softmax(WideTile<NT>& t, const floatx16& s, i
 #pragma unroll
   for (int i = 0; i < 16; ++i) {
     const int key = key_base + pw_key_of(i, g);
-    v[i] = (key >= t.lo && key <= t.hi) ? s[i] : -INFINITY;
+    const float x = MODE == ATTN_SHAPED ? pw_shaped<NT>(t, s[i], i, key_base, g) : s[i];
+    v[i] = (key >= t.lo && key <= t.hi) ? x : -INFINITY;
     mx = fmaxf(mx, v[i]);
   }
   mx = xor32_max(mx) * scale_log2;
@@ -233,7 +243,7 @@ __device__ __forceinline__ void pw_rescale(WideTile<NT>& t, float alpha) {
 
 // One epoch with masks and range checks: steps hsA..hsB are the tile's. s_pend / p_pend as
 // described at the top. k_lds: page j, v_lds: page j - 1.
-template <int NT, bool BIAS>
+template <int NT, int MODE>
 __device__ __forceinline__ void pw_plain_epoch(WideTile<NT>& t, floatx16& s_pend, bf16x8 (&p_pend)[2], int j,
                                                int hsA, int hsB, const uint4* k_lds, const uint4* v_lds,
                                                int kl, int vl, int vl_last, int g, float scale_log2) {
@@ -242,14 +252,14 @@ __device__ __forceinline__ void pw_plain_epoch(WideTile<NT>& t, floatx16& s_pend
   if (h0 >= hsA && h0 <= hsB) pw_values<NT>(t.o, v_lds, vl, vl_last, 0, p_pend);
   if (h1 >= hsA && h1 <= hsB) {
     bf16x8 p[2];
-    if (pw_softmax<NT>(t, s_pend, 32 * h1, g, scale_log2, p, alpha)) pw_rescale<NT>(t, alpha);
+    if (pw_softmax<NT, MODE>(t, s_pend, 32 * h1, g, scale_log2, p, alpha)) pw_rescale<NT>(t, alpha);
     pw_values<NT>(t.o, v_lds, vl, vl_last, 1, p);
   }
   if (h2 >= hsA && h2 <= hsB) {
-    const floatx16 s = pw_scores<NT>(t.qf, k_lds, kl, 0, pw_score_start<BIAS>(t.bias, t.hi, 32 * h2, g));
-    if (pw_softmax<NT>(t, s, 32 * h2, g, scale_log2, p_pend, alpha)) pw_rescale<NT>(t, alpha);
+    const floatx16 s = pw_scores<NT>(t.qf, k_lds, kl, 0, pw_score_start<MODE>(t.bias, t.hi, 32 * h2, g));
+    if (pw_softmax<NT, MODE>(t, s, 32 * h2, g, scale_log2, p_pend, alpha)) pw_rescale<NT>(t, alpha);
   }
-  if (h3 >= hsA && h3 <= hsB) s_pend = pw_scores<NT>(t.qf, k_lds, kl, 1, pw_score_start<BIAS>(t.bias, t.hi, 32 * h3, g));
+  if (h3 >= hsA && h3 <= hsB) s_pend = pw_scores<NT>(t.qf, k_lds, kl, 1, pw_score_start<MODE>(t.bias, t.hi, 32 * h3, g));
 }
 
 // One step of the loop without masks: the softmax of the scores in s_pend (step h) beside
@@ -259,7 +269,7 @@ __device__ __forceinline__ void pw_plain_epoch(WideTile<NT>& t, floatx16& s_pend
 // ahead of its product would stall the wavefront for the LDS latency every time); with STAGE
 // the loads of the next pages are issued then, while the first operand is on its way; then
 // the products, each with its piece of the softmax behind it.
-template <int NT, bool STAGE, bool BIAS>
+template <int NT, bool STAGE, int MODE>
 __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, bf16x8 (&p_pend)[2],
                                              const uint4* k_lds, const uint4* v_lds, int kl, int vl,
                                              int vl_last, int hh, int g, float scale_log2,
@@ -291,9 +301,10 @@ __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, 
   // product; three, 46.8). The softmax is cut into 16 pieces: four of the maximum (the last
   // with the exchange between the halves and the new reference point), eight of two exponentials
   // each, four that round two pairs and add them up; product n of P gets the pieces
-  // ceil(16 n / P) .. ceil(16 (n + 1) / P) - 1.
+  // ceil(16 n / P) .. ceil(16 (n + 1) / P) - 1. Where the scores are shaped, 16 pieces of one score each come first.
   constexpr int P = NT + 2 * DT;
-  floatx16 s_next = pw_score_start<BIAS>(t.bias, t.hi, next_key_base, g);   // the scores of the step at next_key_base
+  constexpr int PIECES = MODE == ATTN_SHAPED ? 32 : 16;
+  floatx16 s_next = pw_score_start<MODE>(t.bias, t.hi, next_key_base, g);   // the scores of the step at next_key_base
   float mx = -INFINITY, m_new = t.m, sum = 0.f;
   bool moved = false;
   float e[16];
@@ -307,8 +318,11 @@ __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, 
       s_next = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[n - 2 * DT], t.qf[n - 2 * DT], s_next, 0, 0, 0);
     }
 #pragma unroll
-    for (int piece = (16 * n + P - 1) / P; piece < (16 * (n + 1) + P - 1) / P; ++piece) {
-      if (piece < 4) {
+    for (int turn = (PIECES * n + P - 1) / P; turn < (PIECES * (n + 1) + P - 1) / P; ++turn) {
+      const int piece = turn - (PIECES - 16);
+      if (piece < 0) {
+        s_pend[turn] = pw_shaped<NT>(t, s_pend[turn], turn, next_key_base - 32, g);
+      } else if (piece < 4) {
 #pragma unroll
         for (int i = 4 * piece; i < 4 * piece + 4; ++i) mx = fmaxf(mx, s_pend[i]);
         if (piece == 3) {
@@ -348,7 +362,7 @@ __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, 
   s_pend = s_next;
 }
 
-template <int NT, bool BIAS>
+template <int NT, int MODE>
 __global__ __launch_bounds__(64 * PW_WAVES) __attribute__((amdgpu_waves_per_eu(2, 2))) void
 attention_prefill_wide_kernel(
     uint16_t* __restrict__ out, const uint16_t* __restrict__ q,
@@ -361,6 +375,7 @@ attention_prefill_wide_kernel(
   constexpr int KP = Pw<NT>::K_PIECES, VP = Pw<NT>::V_PIECES;
   __shared__ uint4 k_lds[2 * KP];
   __shared__ uint4 v_lds[2 * VP];
+  __shared__ float table_lds[MODE == ATTN_SHAPED ? HE_ATTN_TABLE_LDS : 1];
 
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int col = lane & 31, g = lane >> 5;
@@ -401,7 +416,7 @@ attention_prefill_wide_kernel(
   const int64_t k_stride = (int64_t)KVH * he_k_page_elems(HD), v_stride = (int64_t)KVH * he_v_page_elems(HD);
   const uint16_t* kp = kpool + (int64_t)kvh * he_k_page_elems(HD);
   const uint16_t* vp = vpool + (int64_t)kvh * he_v_page_elems(HD);
-  const float scale_log2 = scale * 1.4426950408889634f;
+  const float scale_log2 = MODE == ATTN_SHAPED ? 1.f : scale * PW_LOG2E;
 
   // the workgroup's pages: from the first key its first query sees to its last query
   const int blk_last = start + min(q0 + PW_QUERIES, q_len) - 1;
@@ -432,7 +447,14 @@ attention_prefill_wide_kernel(
   t.lo = attn_first(t.hi, window, ex.chunk);
   t.m = -INFINITY;
   t.l = 0.f;
-  t.bias = BIAS ? ex.slopes[h] / scale : 0.f;
+  t.bias = MODE == ATTN_SLOPES ? ex.slopes[h] / scale : 0.f;
+  if (MODE == ATTN_SHAPED) {
+    t.sh = attn_shape_of(ex, h, scale);
+    const int entries = t.sh.table != nullptr ? ex.table_len : 1;
+    for (int i = threadIdx.x; i < entries; i += 64 * PW_WAVES) table_lds[i] = t.sh.table != nullptr ? t.sh.table[i] * PW_LOG2E : 0.f;
+    t.sh.table = table_lds;      // readable behind the barrier that ends the first page's loads
+    t.sh.last = entries - 1;
+  }
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
@@ -473,7 +495,7 @@ attention_prefill_wide_kernel(
   for (; j < jF0; ++j) {
     if (j + 1 <= pbB) pw_stage<Pw<NT>::K_CHUNKS>(k_base + ((j + 1) & 1) * KP * 16, pw_page(kp, pt[j + 1], num_pages, k_stride, lane), wave);
     if (j <= pbB) pw_stage<Pw<NT>::V_CHUNKS>(v_base + (j & 1) * VP * 16, pw_page(vp, pt[j], num_pages, v_stride, lane), wave);
-    pw_plain_epoch<NT, BIAS>(t, s_pend, p_pend, j, hsA, hsB, k_lds + (j & 1) * KP, v_lds + ((j - 1) & 1) * VP, kl, vl,
+    pw_plain_epoch<NT, MODE>(t, s_pend, p_pend, j, hsA, hsB, k_lds + (j & 1) * KP, v_lds + ((j - 1) & 1) * VP, kl, vl,
                        vl_last, g, scale_log2);
     pw_epoch_end();
   }
@@ -494,8 +516,8 @@ attention_prefill_wide_kernel(
     next.v_src = pw_page(vp, page_v, num_pages, v_stride, lane);   // j <= pbB: the tile's own keys lie beyond step 2j
     const uint4* kb = k_lds + (j & 1) * KP;
     const uint4* vb = v_lds + ((j - 1) & 1) * VP;
-    pw_fast_step<NT, true, BIAS>(t, s_pend, p_pend, kb, vb, kl, vl, vl_last, 0, g, scale_log2, next, wave, 64 * j);
-    pw_fast_step<NT, false, BIAS>(t, s_pend, p_pend, kb, vb, kl, vl, vl_last, 1, g, scale_log2, next, wave, 64 * j + 32);
+    pw_fast_step<NT, true, MODE>(t, s_pend, p_pend, kb, vb, kl, vl, vl_last, 0, g, scale_log2, next, wave, 64 * j);
+    pw_fast_step<NT, false, MODE>(t, s_pend, p_pend, kb, vb, kl, vl, vl_last, 1, g, scale_log2, next, wave, 64 * j + 32);
     // asked for here, not earlier: scalar loads count with the LDS reads, and a wait for an LDS read
     // that follows one would wait for all of them; the barrier below waits for everything anyway
     __builtin_amdgcn_sched_barrier(0);
@@ -506,7 +528,7 @@ attention_prefill_wide_kernel(
   for (; j <= pbB + 1; ++j) {
     if (j + 1 <= pbB) pw_stage<Pw<NT>::K_CHUNKS>(k_base + ((j + 1) & 1) * KP * 16, pw_page(kp, pt[j + 1], num_pages, k_stride, lane), wave);
     if (j <= pbB) pw_stage<Pw<NT>::V_CHUNKS>(v_base + (j & 1) * VP * 16, pw_page(vp, pt[j], num_pages, v_stride, lane), wave);
-    pw_plain_epoch<NT, BIAS>(t, s_pend, p_pend, j, hsA, hsB, k_lds + (j & 1) * KP, v_lds + ((j - 1) & 1) * VP, kl, vl,
+    pw_plain_epoch<NT, MODE>(t, s_pend, p_pend, j, hsA, hsB, k_lds + (j & 1) * KP, v_lds + ((j - 1) & 1) * VP, kl, vl,
                        vl_last, g, scale_log2);
     pw_epoch_end();
   }
@@ -564,11 +586,14 @@ int he_attention_prefill_wide(void* out, const void* q, const void* kpool, const
       (const int32_t*)page_table, max_blocks, num_pages, H, KVH, window, scale, parts, ws_o, ws_ml, ex
 #define PREFILL_WIDE(NTV)                                                                       \
   case NTV:                                                                                     \
-    if (ex.slopes != nullptr)                                                                   \
-      attention_prefill_wide_kernel<NTV, true><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS);  \
+    if (mode == ATTN_SLOPES)                                                                    \
+      attention_prefill_wide_kernel<NTV, ATTN_SLOPES><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
+    else if (mode == ATTN_SHAPED)                                                               \
+      attention_prefill_wide_kernel<NTV, ATTN_SHAPED><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
     else                                                                                        \
-      attention_prefill_wide_kernel<NTV, false><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
+      attention_prefill_wide_kernel<NTV, ATTN_RAW><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
     break;
+  const int mode = attn_mode(ex);
   switch (hd / 16) {
     PREFILL_WIDE(1) PREFILL_WIDE(2) PREFILL_WIDE(3) PREFILL_WIDE(4)
     PREFILL_WIDE(5) PREFILL_WIDE(6) PREFILL_WIDE(7) PREFILL_WIDE(8)

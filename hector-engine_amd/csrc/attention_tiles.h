@@ -38,13 +38,45 @@ __device__ __forceinline__ bf16x8 ld8(const uint16_t* p, bool ok) {
   return __builtin_bit_cast(bf16x8, v);
 }
 
+// What the scores of a kernel pass through (the kernels' template parameter MODE): nothing, a slope over the distance
+// added to the raw score, or a cap and a table over the distance (AttnShape).
+enum { ATTN_RAW = 0, ATTN_SLOPES = 1, ATTN_SHAPED = 2 };
+__host__ __device__ __forceinline__ int attn_mode(const AttnExtras& ex) {
+  return ex.slopes != nullptr ? ATTN_SLOPES : (ex.table != nullptr || ex.cap > 0.f) ? ATTN_SHAPED : ATTN_RAW;
+}
+
+// Raw score s = q . k of a head to the shaped score in the base-2 domain,
+//   log2(e) * (cap * tanh(s * scale / cap) + table[distance]),
+// with tanh(x) = 1 - 2 / (1 + e^(2x)): one exponential and one reciprocal a score (both saturate to the right limits).
+struct AttnShape {
+  float k1;              // capped: 2 log2(e) scale / cap, the exponent's factor; else log2(e) scale
+  float c0, c1;          // capped: log2(e) cap and twice that; else 0
+  const float* table;    // the head's entries, or null
+  int last;              // the table's last index
+};
+__device__ __forceinline__ AttnShape attn_shape_of(const AttnExtras& ex, int h, float scale) {
+  constexpr float L = 1.4426950408889634f;
+  AttnShape a;
+  a.k1 = ex.cap > 0.f ? 2.f * L * scale / ex.cap : L * scale;
+  a.c0 = ex.cap > 0.f ? L * ex.cap : 0.f;
+  a.c1 = 2.f * a.c0;
+  a.table = ex.table != nullptr ? ex.table + (int64_t)h * ex.table_len : nullptr;
+  a.last = ex.table_len - 1;
+  return a;
+}
+__device__ __forceinline__ float attn_cap(const AttnShape& a, float s) {
+  const float x = s * a.k1;
+  return a.c1 > 0.f ? __builtin_fmaf(-a.c1, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x)), a.c0) : x;
+}
+
 template <int NT>
 struct AttnState {
   floatx4 o[NT];  // O^T[16*dt + 4*lg + i][q], unnormalised
   float m;        // reference point (near the running maximum) of the query of this lane's column
   float l;        // this lane's share of the running sum
-  float bias;     // BIAS kernels: the raw score of key j gains bias * (j - pos) (a distance slope over the score scale)
-  int pos;        // BIAS kernels: the position of this lane's query
+  float bias;     // ATTN_SLOPES: the raw score of key j gains bias * (j - pos) (a distance slope over the score scale)
+  int pos;        // ATTN_SLOPES, ATTN_SHAPED: the position of this lane's query
+  AttnShape sh;   // ATTN_SHAPED (its kernels pass scale_log2 = 1: the shaped score is in the base-2 domain already)
 };
 
 // The K and V^T operands of one step of 32 keys, loaded ahead of their use so that the
@@ -84,13 +116,21 @@ __device__ __forceinline__ void load_frag(KVFrag<NT>& f, const uint16_t* __restr
 // base-2 domain: s2 = (q . k) * scale * log2(e), p = 2^(s2 - m), so the exponential is
 // the bare hardware instruction; m is the reference point of s2 (see HE_SOFTMAX_SLACK). When
 // no query's reference point moves, the rescaling of the accumulators is skipped.
-template <int NT, bool MASK, bool BIAS = false>
+template <int NT, bool MASK, int MODE = ATTN_RAW>
 __device__ __forceinline__ void attend_frag(AttnState<NT>& st, const bf16x8* qf,
                                             const KVFrag<NT>& f, int key_base, int lo, int hi,
                                             float scale_log2, int lg) {
   constexpr int HD = 16 * NT;
   constexpr int KS = (HD + 31) / 32;
   if (MASK && !f.ok) hi = -1;
+  float tab[2][4];
+  if (MODE == ATTN_SHAPED && st.sh.table != nullptr) {   // ahead of the products: on their way while those run
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        tab[t][r] = st.sh.table[min(max(st.pos - (key_base + 8 * lg + 4 * t + r), 0), st.sh.last)];
+  }
   floatx4 s[2];
 #pragma unroll
   for (int t = 0; t < 2; ++t) {
@@ -108,7 +148,11 @@ __device__ __forceinline__ void attend_frag(AttnState<NT>& st, const bf16x8* qf,
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       float v = s[t][r];
-      if (BIAS) v = __builtin_fmaf(st.bias, (float)(key_base + 8 * lg + 4 * t + r - st.pos), v);
+      if (MODE == ATTN_SLOPES) v = __builtin_fmaf(st.bias, (float)(key_base + 8 * lg + 4 * t + r - st.pos), v);
+      if (MODE == ATTN_SHAPED) {
+        v = attn_cap(st.sh, v);
+        if (st.sh.table != nullptr) v = __builtin_fmaf(tab[t][r], 1.4426950408889634f, v);
+      }
       if (MASK) {
         const int key = key_base + 8 * lg + 4 * t + r;
         v = (key >= lo && key <= hi) ? v : -INFINITY;
@@ -199,7 +243,7 @@ __device__ __forceinline__ void attend_start(AttendCursor<NT>& c, const uint16_t
 
 // Runs the keys [kb_begin, kb_end) (multiples of 32) of one (sequence, kv head) against the
 // state, one step ahead with its loads and one page ahead with its page-table entry.
-template <int NT, bool UNMASKED_STEPS, bool BIAS = false>
+template <int NT, bool UNMASKED_STEPS, int MODE = ATTN_RAW>
 __device__ __forceinline__ void attend_walk(AttnState<NT>& st, const bf16x8* qf, AttendCursor<NT>& c,
                                             const int32_t* __restrict__ pt, int max_blocks,
                                             int num_pages, int kb_begin, int kb_end, int lo, int hi,
@@ -218,14 +262,14 @@ __device__ __forceinline__ void attend_walk(AttnState<NT>& st, const bf16x8* qf,
     }
     // keys in [clear_lo, clear_hi] are visible to every query of the tile
     if (UNMASKED_STEPS && kb >= clear_lo && kb + 31 <= clear_hi && c.cur.ok)
-      attend_frag<NT, false, BIAS>(st, qf, c.cur, kb, lo, hi, scale_log2, lg);
+      attend_frag<NT, false, MODE>(st, qf, c.cur, kb, lo, hi, scale_log2, lg);
     else
-      attend_frag<NT, true, BIAS>(st, qf, c.cur, kb, lo, hi, scale_log2, lg);
+      attend_frag<NT, true, MODE>(st, qf, c.cur, kb, lo, hi, scale_log2, lg);
     c.cur = nxt;
   }
 }
 
-template <int NT, bool UNMASKED_STEPS, bool BIAS = false>
+template <int NT, bool UNMASKED_STEPS, int MODE = ATTN_RAW>
 __device__ __forceinline__ void attend_range(AttnState<NT>& st, const bf16x8* qf,
                                              const uint16_t* __restrict__ kpool,
                                              const uint16_t* __restrict__ vpool,
@@ -236,7 +280,7 @@ __device__ __forceinline__ void attend_range(AttnState<NT>& st, const bf16x8* qf
   if (kb_begin >= kb_end) return;
   AttendCursor<NT> c;
   attend_start<NT>(c, kpool, vpool, pt, max_blocks, num_pages, KVH, kvh, kb_begin, lr, lg);
-  attend_walk<NT, UNMASKED_STEPS, BIAS>(st, qf, c, pt, max_blocks, num_pages, kb_begin, kb_end, lo, hi,
+  attend_walk<NT, UNMASKED_STEPS, MODE>(st, qf, c, pt, max_blocks, num_pages, kb_begin, kb_end, lo, hi,
                                   clear_lo, clear_hi, scale_log2, lr, lg);
 }
 

@@ -177,18 +177,22 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   return total;
 }
 
-// A gated activation's constants: out = g' * sigmoid(alpha g') * (u' + shift) with g' = min(g, limit),
+// A gated activation's constants: out = g' * sigmoid(alpha g' + cubic g'^3) * (u' + shift) with g' = min(g, limit),
 // u' = clamp(u, -limit, limit) (limit +inf: unbounded). CLAMPED false is SiLU(g) * u, written as it
-// always was (the constants are then not read).
+// always was (the constants are then not read). The tanh form of gelu is one of them:
+// 0.5 g (1 + tanh(c (g + a g^3))) = g * sigmoid(2 c g + 2 c a g^3).
 struct GatedAct {
-  float alpha, limit, shift;
+  float alpha, limit, shift, cubic;
 };
+inline bool he_gated_act_is_silu(float alpha, float limit, float shift, float cubic) {
+  return alpha == 1.f && !(limit > 0.f) && shift == 0.f && cubic == 0.f;
+}
 template <bool CLAMPED>
 __device__ __forceinline__ float he_gated_act(float g, float u, const GatedAct& a) {
   if (!CLAMPED) return g / (1.f + expf(-g)) * u;
   g = fminf(g, a.limit);
   u = fminf(fmaxf(u, -a.limit), a.limit);
-  return g / (1.f + expf(-a.alpha * g)) * (u + a.shift);
+  return g / (1.f + expf(-fmaf(a.cubic, g * g, a.alpha) * g)) * (u + a.shift);
 }
 
 // tanh for a result that is rounded to bfloat16: (1 - t) / (1 + t) with t = exp(-2 |z|), the sign put back
@@ -214,7 +218,8 @@ int he_cus();
 // null or zero: chunk > 0, a query sees no key before the start of its own chunk of that many
 // positions (counted from position 0); sinks, a number a head that joins the softmax's denominator
 // as exp(sink) without a key or value (not scaled); gate, gate[row * gate_stride + h] (bf16), whose
-// sigmoid multiplies the head's output.
+// sigmoid multiplies the head's output; cap and table shape the scores: with cap > 0 a score s becomes
+// cap * tanh(s / cap), and then gains table[h][min(p - j, table_len - 1)] for key j and the query at p.
 struct AttnExtras {
   const void* sinks;
   int sinks_dtype;
@@ -222,6 +227,9 @@ struct AttnExtras {
   int64_t gate_stride;
   int chunk;
   const float* slopes;   // [H] or null: the score of key j for the query at p loses slopes[h] * (p - j)
+  const float* table;    // [H][table_len] or null: what a score gains at each distance (the last entry: and beyond)
+  int table_len;
+  float cap;             // 0: scores are not capped
 };
 // attention_mfma.hip: joins attention parts that were all stored (the fused one-token kernel's, the
 // prompt kernel's); row_seq may be null: every row has a sequence

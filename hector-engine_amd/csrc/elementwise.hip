@@ -81,16 +81,20 @@ extern "C" int he_gather_rows_f32(void* out, const void* src, const void* rows, 
   return he_check_launch("he_gather_rows_f32");
 }
 
-// resid[r, :] += scale * delta[r, :], the residual sum in fp32 (scale 1: the plain sum).
+// resid[r, :] += scale * (delta[r, :] + delta2[r, :]), the residual sum in fp32 (scale 1: the plain sum; delta2 may be null).
 template <typename T>
 __global__ void residual_add_kernel(float* __restrict__ resid, const T* __restrict__ delta,
-                                    int64_t n, float scale) {
+                                    const T* __restrict__ delta2, int64_t n, float scale) {
   int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
   const int64_t stride = (int64_t)gridDim.x * blockDim.x;
+  if (delta2 != nullptr) {
+    for (; i < n; i += stride) resid[i] += scale * (to_float(delta[i]) + to_float(delta2[i]));
+    return;
+  }
   for (; i < n; i += stride) resid[i] += scale * to_float(delta[i]);
 }
 
-extern "C" int he_residual_add(void* resid_f32, const void* delta, int64_t n, int delta_dtype,
+extern "C" int he_residual_add(void* resid_f32, const void* delta, const void* delta2, int64_t n, int delta_dtype,
                                float scale, void* stream) {
   HE_REQUIRE(n >= 0, "he_residual_add: bad size");
   if (n == 0) return 0;
@@ -99,10 +103,10 @@ extern "C" int he_residual_add(void* resid_f32, const void* delta, int64_t n, in
   hipStream_t s = (hipStream_t)stream;
   if (delta_dtype == HE_BF16)
     residual_add_kernel<bf16_t><<<(int)blocks, 256, 0, s>>>((float*)resid_f32,
-                                                            (const bf16_t*)delta, n, scale);
+                                                            (const bf16_t*)delta, (const bf16_t*)delta2, n, scale);
   else if (delta_dtype == HE_F32)
     residual_add_kernel<float><<<(int)blocks, 256, 0, s>>>((float*)resid_f32, (const float*)delta,
-                                                           n, scale);
+                                                           (const float*)delta2, n, scale);
   else
     HE_REQUIRE(false, "he_residual_add: unknown dtype %d", delta_dtype);
   return he_check_launch("he_residual_add");
@@ -210,9 +214,9 @@ static int gated_act_launch(void* out, const void* gate_up, int rows, int I, int
 
 // out = act(gate) * up over gate||up columns as he_silu_mul takes them, with
 // gate' = min(gate, limit), up' = clamp(up, -limit, limit) (limit <= 0: neither is bounded),
-// out = gate' * sigmoid(alpha * gate') * (up' + up_shift). alpha 1, no limit and no shift is SiLU(gate) * up.
+// out = gate' * sigmoid(alpha * gate' + cubic * gate'^3) * (up' + up_shift). alpha 1 and the rest 0 is SiLU(gate) * up.
 extern "C" int he_gated_act(void* out, const void* gate_up, int rows, int I, int interleaved, int splits,
-                            int dtype, float alpha, float limit, float up_shift, void* stream) {
+                            int dtype, float alpha, float limit, float up_shift, float cubic, void* stream) {
   HE_REQUIRE(rows >= 0 && I > 0, "he_gated_act: bad sizes rows=%d I=%d", rows, I);
   HE_REQUIRE(splits >= 0 && splits <= 64, "he_gated_act: bad slice count %d", splits);
   HE_REQUIRE(dtype == HE_BF16 || dtype == HE_F32, "he_gated_act: unknown dtype %d", dtype);
@@ -221,14 +225,15 @@ extern "C" int he_gated_act(void* out, const void* gate_up, int rows, int I, int
   act.alpha = alpha;
   act.limit = limit > 0.f ? limit : INFINITY;
   act.shift = up_shift;
-  if (alpha == 1.f && !(limit > 0.f) && up_shift == 0.f)
+  act.cubic = cubic;
+  if (he_gated_act_is_silu(alpha, limit, up_shift, cubic))
     return gated_act_launch<false>(out, gate_up, rows, I, interleaved, splits, dtype, act, (hipStream_t)stream);
   return gated_act_launch<true>(out, gate_up, rows, I, interleaved, splits, dtype, act, (hipStream_t)stream);
 }
 
 extern "C" int he_silu_mul(void* out, const void* gate_up, int rows, int I, int interleaved,
                            int splits, int dtype, void* stream) {
-  return he_gated_act(out, gate_up, rows, I, interleaved, splits, dtype, 1.f, 0.f, 0.f, stream);
+  return he_gated_act(out, gate_up, rows, I, interleaved, splits, dtype, 1.f, 0.f, 0.f, 0.f, stream);
 }
 
 // ---- activations and gates of one input -----------------------------------------------------------

@@ -124,7 +124,7 @@ extern "C" int he_gemm_blocksplit_fused_bf16(void* C, const void* A, const void*
                                              float scale_eps, void* resid, const void* gain,
                                              int gain_dtype, void* xg, void* sq_out,
                                              int sq_count, int x_pieces, int out_pieces,
-                                             float act_alpha, float act_limit, float act_shift,
+                                             float act_alpha, float act_limit, float act_shift, float act_cubic,
                                              float resid_scale, const void* dyt_bias,
                                              const void* dyt_alpha, void* stream) {
   HE_REQUIRE((dyt_alpha == nullptr) == (dyt_bias == nullptr), "he_gemm_blocksplit_bf16: Dynamic Tanh needs alpha and bias");
@@ -168,10 +168,11 @@ extern "C" int he_gemm_blocksplit_fused_bf16(void* C, const void* A, const void*
   fu.xg = (uint16_t*)xg;
   fu.sq_out = (float*)sq_out;
   fu.out_pieces = out_pieces;
-  fu.act_clamped = gated && !(act_alpha == 1.f && !(act_limit > 0.f) && act_shift == 0.f);
+  fu.act_clamped = gated && !he_gated_act_is_silu(act_alpha, act_limit, act_shift, act_cubic);
   fu.act.alpha = act_alpha;
   fu.act.limit = act_limit > 0.f ? act_limit : INFINITY;
   fu.act.shift = act_shift;
+  fu.act.cubic = act_cubic;
   fu.resid_scale = resid_scale;
   fu.dyt_bias = dyt_bias;
   fu.dyt_alpha = dyt_alpha;
@@ -190,5 +191,5 @@ extern "C" int he_gemm_blocksplit_bf16(void* C, const void* A, const void* W, co
                                        int gated, int R, int U, int NW, void* stream) {
   return he_gemm_blocksplit_fused_bf16(C, A, W, bias, M, N, K, out_dtype, bias_dtype, gated, R, U,
                                        NW, nullptr, 0, 0.f, nullptr, nullptr, HE_F32, nullptr,
-                                       nullptr, 0, 0, 0, 1.f, 0.f, 0.f, 1.f, nullptr, nullptr, stream);
+                                       nullptr, 0, 0, 0, 1.f, 0.f, 0.f, 0.f, 1.f, nullptr, nullptr, stream);
 }

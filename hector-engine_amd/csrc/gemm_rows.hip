@@ -85,7 +85,7 @@ extern "C" int he_gemm_rows_bf16(void* C, void* partial_f32, int64_t partial_flo
                                  const void* scale_partials, int scale_count, float scale_eps,
                                  void* resid, const void* gain, int gain_dtype, void* xg, void* sq_out,
                                  int sq_count, int x_pieces, int out_pieces, int* splits_used,
-                                 float act_alpha, float act_limit, float act_shift, float resid_scale,
+                                 float act_alpha, float act_limit, float act_shift, float act_cubic, float resid_scale,
                                  const void* dyt_bias, const void* dyt_alpha, void* stream) {
   HE_REQUIRE((dyt_alpha == nullptr) == (dyt_bias == nullptr), "he_gemm_rows_bf16: Dynamic Tanh needs alpha and bias");
   HE_REQUIRE(M > 0 && M <= HE_GEMM_ROWS_MAX_M, "he_gemm_rows_bf16: M=%d outside [1, %d]", M,
@@ -135,10 +135,11 @@ extern "C" int he_gemm_rows_bf16(void* C, void* partial_f32, int64_t partial_flo
   fu.xg = (uint16_t*)xg;
   fu.sq_out = (float*)sq_out;
   fu.out_pieces = out_pieces;
-  fu.act_clamped = gated && !(act_alpha == 1.f && !(act_limit > 0.f) && act_shift == 0.f);
+  fu.act_clamped = gated && !he_gated_act_is_silu(act_alpha, act_limit, act_shift, act_cubic);
   fu.act.alpha = act_alpha;
   fu.act.limit = act_limit > 0.f ? act_limit : INFINITY;
   fu.act.shift = act_shift;
+  fu.act.cubic = act_cubic;
   fu.resid_scale = resid_scale;
   fu.dyt_bias = dyt_bias;
   fu.dyt_alpha = dyt_alpha;

@@ -6,7 +6,7 @@
 #pragma once
 #include <stdint.h>
 
-#define HE_ABI_VERSION 29
+#define HE_ABI_VERSION 30
 
 #ifdef __cplusplus
 extern "C" {
@@ -31,26 +31,26 @@ int he_embedding(void* out_f32, const void* table, const void* ids, int rows, in
                  int table_dtype, float scale, void* stream);
 int he_gather_rows_f32(void* out, const void* src, const void* rows, int n_out, int D, int n_src,
                        void* stream);
-// resid += scale * delta.
-int he_residual_add(void* resid_f32, const void* delta, int64_t n, int delta_dtype, float scale,
+// resid += scale * (delta + delta2) (delta2 may be null).
+int he_residual_add(void* resid_f32, const void* delta, const void* delta2, int64_t n, int delta_dtype, float scale,
                     void* stream);
 // splits > 0: gate_up is fp32 [splits][rows][2I], the K slices of the product.
 int he_silu_mul(void* out, const void* gate_up, int rows, int I, int interleaved, int splits,
                 int dtype, void* stream);
 // The same columns through a gated activation with constants: gate' = min(gate, limit),
-// up' = clamp(up, -limit, limit) (limit <= 0: unbounded), out = gate' * sigmoid(alpha * gate') *
-// (up' + up_shift). alpha 1 without limit and shift is he_silu_mul.
+// up' = clamp(up, -limit, limit) (limit <= 0: unbounded), out = gate' * sigmoid(alpha * gate' + cubic * gate'^3) *
+// (up' + up_shift). alpha 1 without limit, shift and cubic term is he_silu_mul.
 int he_gated_act(void* out, const void* gate_up, int rows, int I, int interleaved, int splits,
-                 int dtype, float alpha, float limit, float up_shift, void* stream);
+                 int dtype, float alpha, float limit, float up_shift, float cubic, void* stream);
 
 // ---- norms ---------------------------------------------------------------
 // resid (fp32, in place) += delta (may be null); out (may be null) = rmsnorm(resid) * weight.
 int he_add_rmsnorm(void* resid_f32, const void* delta, const void* weight, void* out, int rows, int D,
                    float eps, int act_dtype, int w_dtype, void* stream);
-// Dynamic Tanh where a norm would stand: resid (fp32, in place) += delta_scale * delta (may be null);
+// Dynamic Tanh where a norm would stand: resid (fp32, in place) += delta_scale * (delta + delta2) (may be null, delta2 alone too);
 // out (may be null) = tanh(alpha * resid) * weight + bias, alpha a stored scalar (device pointer),
 // weight and bias vectors [D], all three of w_dtype.
-int he_add_dyt(void* resid_f32, const void* delta, float delta_scale, const void* weight,
+int he_add_dyt(void* resid_f32, const void* delta, const void* delta2, float delta_scale, const void* weight,
                const void* bias, const void* alpha, void* out, int rows, int D, int act_dtype,
                int w_dtype, void* stream);
 int he_rmsnorm_rows(void* out, const void* x, const void* weight, int rows, int D,
@@ -88,15 +88,15 @@ int he_gemm_blocksplit_fused_bf16(void* C, const void* A, const void* W, const v
                                   int U, int NW, const void* scale_partials, int scale_count,
                                   float scale_eps, void* resid, const void* gain, int gain_dtype,
                                   void* xg, void* sq_out, int sq_count, int x_pieces, int out_pieces,
-                                  float act_alpha, float act_limit, float act_shift, float resid_scale,
+                                  float act_alpha, float act_limit, float act_shift, float act_cubic, float resid_scale,
                                   const void* dyt_bias, const void* dyt_alpha, void* stream);
 // resid_scale: the residual epilogue adds resid_scale * result. dyt_alpha, dyt_bias (both null, or both
 // of gain's dtype; alpha one stored number): the norm that follows is Dynamic Tanh, and the epilogue
 // leaves it finished, xg = tanh(alpha * resid) * gain + dyt_bias, with sq_out = 0 (a reader that
 // applies 1/sqrt(sum / K + eps) with eps = 1 applies 1). So for he_gemm_rows_bf16 and
 // he_splitk_reduce_residual.
-// act_alpha, act_limit, act_shift: the constants of the gated epilogue as he_gated_act takes them
-// (1, 0, 0: SiLU(gate) * up); so for he_gemm_rows_bf16.
+// act_alpha, act_limit, act_shift, act_cubic: the constants of the gated epilogue as he_gated_act takes them
+// (1, 0, 0, 0: SiLU(gate) * up); so for he_gemm_rows_bf16.
 // out = x / sqrt(sum(partials of the row)/D + eps): such xg rows as a normalised tensor
 // (row-major; x_pieces: x lies piece-major for exactly `rows` rows).
 int he_scale_rows_bf16(void* out, const void* x, const void* partials, int count, int rows, int D,
@@ -118,7 +118,7 @@ int he_gemm_rows_bf16(void* C, void* partial_f32, int64_t partial_floats, const 
                       int R, int NWV, int splits, const void* scale_partials, int scale_count,
                       float scale_eps, void* resid, const void* gain, int gain_dtype, void* xg,
                       void* sq_out, int sq_count, int x_pieces, int out_pieces, int* splits_used,
-                      float act_alpha, float act_limit, float act_shift, float resid_scale,
+                      float act_alpha, float act_limit, float act_shift, float act_cubic, float resid_scale,
                       const void* dyt_bias, const void* dyt_alpha, void* stream);
 // resid[M,N] (fp32, in place) += the slices of partial_f32 [splits][M][N] in index order (+ bias);
 // xg = bf16(resid * gain) (piece-major with out_pieces); sq_out[M, sq_count] = sums of resid^2 per
@@ -162,8 +162,10 @@ int he_attention_plain(void* out, const void* q, const void* kpool, const void* 
                        int KVH, int hd, int window, int chunk, float scale, const void* sinks,
                        int sinks_dtype, const void* gate, int64_t gate_stride, int dtype,
                        int most_keys, void* workspace_f32, int64_t workspace_floats, const void* slopes_f32,
-                       void* stream);
+                       const void* table_f32, int table_len, float cap, void* stream);
 // slopes_f32 (or null): one number a head; the score of key j for the query at p loses slope * (p - j).
+// cap > 0: a score s becomes cap * tanh(s / cap); table_f32 (or null): [H][table_len], the score then gains the
+// entry min(p - j, table_len - 1) of its head. (Slopes and table exclude each other.)
 // bf16, one query row per sequence (decode): split over the keys, then merged. chunk, sinks and
 // gate (bf16 here) as he_attention_plain takes them; so does he_attention_prefill_bf16.
 int he_attention_decode_bf16(void* out, const void* q, const void* kpool, const void* vpool,
@@ -172,7 +174,7 @@ int he_attention_decode_bf16(void* out, const void* q, const void* kpool, const 
                              int H, int KVH, int hd, int window, float scale, int max_keys,
                              void* workspace_f32, int64_t workspace_floats, int chunk,
                              const void* sinks, int sinks_dtype, const void* gate, int64_t gate_stride,
-                             const void* slopes_f32, void* stream);
+                             const void* slopes_f32, const void* table_f32, int table_len, float cap, void* stream);
 int64_t he_attention_decode_workspace_floats(int rows, int H, int KVH, int hd, int max_keys);
 // bf16, one query row per sequence, one launch for bias + rotary + cache write + attention +
 // merge (a second launch joins the parts where few sequences are cut across workgroups).
@@ -213,7 +215,10 @@ int he_attention_prefill_bf16(void* out, const void* q, const void* kpool, const
                               int max_q_len, int H, int KVH, int hd, int window, float scale,
                               int kernel, int total_rows, int parts, void* workspace_f32,
                               int64_t workspace_floats, int chunk, const void* sinks, int sinks_dtype,
-                              const void* gate, int64_t gate_stride, const void* slopes_f32, void* stream);
+                              const void* gate, int64_t gate_stride, const void* slopes_f32,
+                              const void* table_f32, int table_len, float cap, void* stream);
+// the longest distance table kernel 2 takes (it keeps the head's entries in LDS)
+#define HE_ATTN_TABLE_LDS 2048
 
 // ---- state-space mixer (state_space.hip) ------------------------------------
 // A sequence's row of the state area holds, in fp32, the last K-1 inputs of the convolution [K-1][C] at
@@ -258,18 +263,22 @@ int he_mlstm_scan(void* y_f32, const void* q, const void* k, const void* v, int6
 int he_route_tokens(void* dense_f32, void* ids_i32, void* weights_f32, const void* logits_f32,
                     const void* x, int x_dtype, const void* router_f32, int D,
                     const void* correction, int c_dtype, int rows, int E, int real, int groups, int keep,
-                    int top, float scale, int normalize, void* stream);
+                    int top, float scale, int normalize, const void* bias, int bias_dtype, int x_pieces, void* stream);
+// bias (or null): [E], added to the logits before anything else; x_pieces: the bf16 rows x lie piece-major for exactly `rows` rows.
+// he_routed_act: `shared` more columns behind the experts' (an expert every row uses): weight 1.
 int he_routed_act(void* out, const void* gate_up, const void* dense_f32, const void* h, int rows, int real,
-                  int I, int extra, int dtype, float alpha, float limit, float up_shift, void* stream);
+                  int I, int shared, int extra, int dtype, float alpha, float limit, float up_shift, float cubic,
+                  void* stream);
 // For a step of very few rows (bf16): out[rows][D] = the weighted sum of the chosen experts' results alone, from
 // the same fused matrices the products over all experts use (gate_up [2 real I][D], rows alternating gate and up;
 // down [D][ldw] with the experts' matrices side by side), plus dense[row][real] * x (the identity experts' share).
-// ids / weights [rows][top] and dense [rows][real + 1] as he_route_tokens leaves them; h_scratch: rows * top * I
-// elements. I, D and ldw in multiples of 8.
+// ids / weights [rows][top] and dense [rows][real + 1] as he_route_tokens leaves them; h_scratch: rows * (top * I + shared)
+// elements. I, D, shared and ldw in multiples of 8. shared: columns behind the experts' that every row uses with weight 1.
+// x_pieces: x lies piece-major (no identity share then).
 int he_chosen_experts(void* out, void* h_scratch, const void* x, const void* gate_up, const void* down,
                       int64_t ldw, const void* ids_i32, const void* weights_f32, const void* dense_f32,
-                      int rows, int top, int real, int I, int D, float alpha, float limit, float up_shift,
-                      void* stream);
+                      int rows, int top, int real, int I, int shared, int D, float alpha, float limit, float up_shift,
+                      float cubic, int x_pieces, void* stream);
 int he_diff_heads(void* out, const void* attn, int rows, int H, int G, int hd, int vd, float lambda,
                   float post, float eps, int dtype, void* stream);
 
@@ -360,9 +369,17 @@ int he_gated_add(void* out, const void* a, const void* b, const void* x, const v
 // ---- latent attention (latent.hip) ---------------------------------------------------------------------
 // out[r, h, n] = sum_k x[r, h, k] w[h][k][n]
 int he_head_product(void* out, int64_t o_row, int64_t o_head, const void* x, int64_t x_row, int64_t x_head, const void* w,
-                    int w_dtype, int rows, int H, int K, int N, int dtype, void* stream);
-int he_latent_pack(void* qkv, const void* q, const void* down, int64_t down_stride, int rows, int H, int d, int r,
-                   int rank, int dtype, void* stream);
+                    int w_dtype, int rows, int H, int K, int N, const void* gate, int64_t gate_row, int dtype,
+                    void* stream);
+// The same products on the matrix cores: bf16, w [H][N][K] (K in multiples of 8), x rows and heads on 16-byte boundaries.
+// gate (or null; both forms): out *= sigmoid(gate[r * gate_row + h * N + n]).
+int he_head_product_mfma(void* out, int64_t o_row, int64_t o_head, const void* x, int64_t x_row, int64_t x_head, const void* w,
+                         int rows, int H, int K, int N, const void* gate, int64_t gate_row, void* stream);
+int he_latent_cache(void* q_out, int64_t q_out_row, void* kpool, void* vpool, const void* q, int64_t q_row, const void* down,
+                    int64_t down_row, const void* gain, int gain_dtype, float eps, const void* positions,
+                    const void* row_seq, const void* seq_slot, const void* page_table, int max_blocks, int num_pages,
+                    const void* inv_freq, int interleaved, float mscale, int rows, int H, int d, int r, int rank, int pd,
+                    int dtype, void* stream);
 
 #ifdef __cplusplus
 }

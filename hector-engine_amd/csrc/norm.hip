@@ -333,7 +333,8 @@ extern "C" int he_scale_rows_bf16(void* out, const void* x, const void* partials
 // above, it first adds the pending branch output: r = resid + delta_scale * delta (fp32, stored
 // back as the new residual). alpha is read from device memory (a stored tensor of one element).
 template <typename TD, typename TO, typename TW, int VEC>
-__global__ void add_dyt_kernel(float* __restrict__ resid, const TD* __restrict__ delta, float delta_scale,
+__global__ void add_dyt_kernel(float* __restrict__ resid, const TD* __restrict__ delta, const TD* __restrict__ delta2,
+                               float delta_scale,
                                const TW* __restrict__ w, const TW* __restrict__ b,
                                const TW* __restrict__ alpha_p, TO* __restrict__ out, int64_t n, int D) {
   const float alpha = to_float(alpha_p[0]);
@@ -341,10 +342,11 @@ __global__ void add_dyt_kernel(float* __restrict__ resid, const TD* __restrict__
   const int64_t stride = (int64_t)gridDim.x * blockDim.x * VEC;
   for (; i < n; i += stride) {
     const int c = (int)(i % D);
-    float v[VEC], a[VEC], g[VEC], s[VEC];
+    float v[VEC], a[VEC], a2[VEC], g[VEC], s[VEC];
     if constexpr (VEC == 4) {
       load4(resid + i, v);
       if (delta) load4(delta + i, a);
+      if (delta2) load4(delta2 + i, a2);
       if (out) {
         load4(w + c, g);
         load4(b + c, s);
@@ -352,9 +354,14 @@ __global__ void add_dyt_kernel(float* __restrict__ resid, const TD* __restrict__
     } else {
       v[0] = resid[i];
       if (delta) a[0] = to_float(delta[i]);
+      if (delta2) a2[0] = to_float(delta2[i]);
       if (out) g[0] = to_float(w[c]), s[0] = to_float(b[c]);
     }
     if (delta) {
+      if (delta2) {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) a[j] += a2[j];
+      }
 #pragma unroll
       for (int j = 0; j < VEC; ++j) v[j] = fmaf(delta_scale, a[j], v[j]);
       if constexpr (VEC == 4) store4(resid + i, v);
@@ -371,33 +378,34 @@ __global__ void add_dyt_kernel(float* __restrict__ resid, const TD* __restrict__
 }
 
 template <typename TD, typename TO, typename TW>
-static void launch_add_dyt(float* resid, const void* delta, float delta_scale, const void* w, const void* b,
+static void launch_add_dyt(float* resid, const void* delta, const void* delta2, float delta_scale, const void* w, const void* b,
                            const void* alpha, void* out, int rows, int D, hipStream_t s) {
   const int64_t n = (int64_t)rows * D;
-  const bool vec = (D & 3) == 0 && ((((uintptr_t)resid) | ((uintptr_t)delta) | ((uintptr_t)w) | ((uintptr_t)b) |
+  const bool vec = (D & 3) == 0 && ((((uintptr_t)resid) | ((uintptr_t)delta) | ((uintptr_t)delta2) | ((uintptr_t)w) | ((uintptr_t)b) |
                                      ((uintptr_t)out)) & 15) == 0;
   const int64_t items = vec ? n / 4 : n;
   int64_t blocks = (items + 255) / 256;
   if (blocks > 65535 * 16) blocks = 65535 * 16;
   if (vec)
-    add_dyt_kernel<TD, TO, TW, 4><<<(unsigned)blocks, 256, 0, s>>>(resid, (const TD*)delta, delta_scale, (const TW*)w,
+    add_dyt_kernel<TD, TO, TW, 4><<<(unsigned)blocks, 256, 0, s>>>(resid, (const TD*)delta, (const TD*)delta2, delta_scale, (const TW*)w,
                                                                    (const TW*)b, (const TW*)alpha, (TO*)out, n, D);
   else
-    add_dyt_kernel<TD, TO, TW, 1><<<(unsigned)blocks, 256, 0, s>>>(resid, (const TD*)delta, delta_scale, (const TW*)w,
+    add_dyt_kernel<TD, TO, TW, 1><<<(unsigned)blocks, 256, 0, s>>>(resid, (const TD*)delta, (const TD*)delta2, delta_scale, (const TW*)w,
                                                                    (const TW*)b, (const TW*)alpha, (TO*)out, n, D);
 }
 
-extern "C" int he_add_dyt(void* resid_f32, const void* delta, float delta_scale, const void* weight,
+extern "C" int he_add_dyt(void* resid_f32, const void* delta, const void* delta2, float delta_scale, const void* weight,
                           const void* bias, const void* alpha, void* out, int rows, int D, int act_dtype,
                           int w_dtype, void* stream) {
   HE_REQUIRE(rows >= 0 && D > 0, "he_add_dyt: bad sizes rows=%d D=%d", rows, D);
   HE_REQUIRE(w_dtype == HE_F32 || w_dtype == HE_BF16, "he_add_dyt: bad parameter dtype");
   HE_REQUIRE(act_dtype == HE_F32 || act_dtype == HE_BF16, "he_add_dyt: unknown dtype %d", act_dtype);
   HE_REQUIRE(out == nullptr || (weight && bias && alpha), "he_add_dyt: weight, bias and alpha are needed");
+  HE_REQUIRE(delta2 == nullptr || delta != nullptr, "he_add_dyt: delta2 goes with delta");
   if (rows == 0 || (delta == nullptr && out == nullptr)) return 0;
   hipStream_t s = (hipStream_t)stream;
   float* r = (float*)resid_f32;
-#define DYT(TD, TO, TW) launch_add_dyt<TD, TO, TW>(r, delta, delta_scale, weight, bias, alpha, out, rows, D, s)
+#define DYT(TD, TO, TW) launch_add_dyt<TD, TO, TW>(r, delta, delta2, delta_scale, weight, bias, alpha, out, rows, D, s)
   if (act_dtype == HE_BF16) {
     if (w_dtype == HE_BF16) DYT(bf16_t, bf16_t, bf16_t);
     else DYT(bf16_t, bf16_t, float);

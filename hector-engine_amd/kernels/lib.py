@@ -16,7 +16,7 @@ _lib = None
 
 _CSRC = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "csrc")
 
-EXPECTED_ABI = 29
+EXPECTED_ABI = 30
 
 c_int, c_i64, c_f32, c_ptr = ctypes.c_int, ctypes.c_int64, ctypes.c_float, ctypes.c_void_p
 
@@ -28,10 +28,10 @@ _SIGNATURES = {
     "he_cast": [c_ptr, c_ptr, c_i64, c_int, c_int, c_ptr],
     "he_embedding": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_f32, c_ptr],
     "he_gather_rows_f32": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_ptr],
-    "he_residual_add": [c_ptr, c_ptr, c_i64, c_int, c_f32, c_ptr],
+    "he_residual_add": [c_ptr, c_ptr, c_ptr, c_i64, c_int, c_f32, c_ptr],
     "he_silu_mul": [c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_ptr],
-    "he_gated_act": [c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_ptr],
-    "he_add_dyt": [c_ptr, c_ptr, c_f32, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_ptr],
+    "he_gated_act": [c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_f32, c_ptr],
+    "he_add_dyt": [c_ptr, c_ptr, c_ptr, c_f32, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_ptr],
     "he_add_rmsnorm": [c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_f32, c_int, c_int, c_ptr],
     "he_rmsnorm_rows": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_i64, c_i64, c_f32, c_int, c_int, c_ptr],
     "he_gemm_plain_workspace_floats": [c_int, c_int, c_int],
@@ -42,14 +42,14 @@ _SIGNATURES = {
     "he_gemm_blocksplit_blocks": [c_int, c_int, c_int],
     "he_gemm_blocksplit_fused_bf16": [c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_int,
                                       c_int, c_int, c_int, c_ptr, c_int, c_f32, c_ptr, c_ptr, c_int,
-                                      c_ptr, c_ptr, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_f32, c_ptr, c_ptr,
+                                      c_ptr, c_ptr, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_f32, c_f32, c_ptr, c_ptr,
                                       c_ptr],
     "he_scale_rows_bf16": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_f32, c_int, c_ptr],
     "he_splitk_reduce": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_ptr],
     "he_gemm_rows_plan": [c_int, c_int, c_int, ctypes.POINTER(c_int), ctypes.POINTER(c_int)],
     "he_gemm_rows_bf16": [c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_int,
                           c_int, c_int, c_int, c_ptr, c_int, c_f32, c_ptr, c_ptr, c_int, c_ptr, c_ptr, c_int,
-                          c_int, c_int, ctypes.POINTER(c_int), c_f32, c_f32, c_f32, c_f32, c_ptr, c_ptr, c_ptr],
+                          c_int, c_int, ctypes.POINTER(c_int), c_f32, c_f32, c_f32, c_f32, c_f32, c_ptr, c_ptr, c_ptr],
     "he_splitk_reduce_residual_blocks": [c_int],
     "he_splitk_reduce_residual": [c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_int, c_ptr, c_ptr, c_int, c_int, c_int,
                                   c_int, c_int, c_f32, c_ptr, c_ptr, c_ptr],
@@ -74,7 +74,7 @@ _SIGNATURES = {
     "he_sigmoid_gate": [c_ptr, c_ptr, c_i64, c_int, c_int, c_int, c_int, c_f32, c_int, c_ptr],
     "he_scaled_sum": [c_ptr, c_ptr, c_ptr, c_i64, c_f32, c_f32, c_int, c_ptr],
     "he_route_tokens": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_int, c_ptr, c_int, c_int, c_int, c_int,
-                        c_int, c_int, c_int, c_f32, c_int, c_ptr],
+                        c_int, c_int, c_int, c_f32, c_int, c_ptr, c_int, c_int, c_ptr],
     "he_delta_state_floats": [c_int, c_int, c_int],
     "he_delta_scan": [c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_i64, c_i64, c_ptr, c_ptr,
                       c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_ptr, c_i64, c_int, c_ptr],
@@ -85,19 +85,23 @@ _SIGNATURES = {
     "he_qk_head_norm": [c_ptr, c_i64, c_ptr, c_i64, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_f32, c_int, c_int, c_int, c_ptr],
     "he_depth_mix": [c_ptr, c_ptr, c_i64, c_ptr, c_int, c_int, c_i64, c_ptr],
     "he_gated_add": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_ptr],
-    "he_head_product": [c_ptr, c_i64, c_i64, c_ptr, c_i64, c_i64, c_ptr, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr],
-    "he_latent_pack": [c_ptr, c_ptr, c_ptr, c_i64, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr],
-    "he_routed_act": [c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_ptr],
+    "he_head_product": [c_ptr, c_i64, c_i64, c_ptr, c_i64, c_i64, c_ptr, c_int, c_int, c_int, c_int, c_int, c_ptr, c_i64,
+                        c_int, c_ptr],
+    "he_head_product_mfma": [c_ptr, c_i64, c_i64, c_ptr, c_i64, c_i64, c_ptr, c_int, c_int, c_int, c_int, c_ptr, c_i64, c_ptr],
+    "he_latent_cache": [c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_i64, c_ptr, c_int, c_f32, c_ptr, c_ptr, c_ptr, c_ptr,
+                        c_int, c_int, c_ptr, c_int, c_f32, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr],
+    "he_routed_act": [c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_f32,
+                      c_ptr],
     "he_chosen_experts": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int,
-                          c_int, c_f32, c_f32, c_f32, c_ptr],
+                          c_int, c_int, c_f32, c_f32, c_f32, c_f32, c_int, c_ptr],
     "he_diff_heads": [c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_f32, c_int, c_ptr],
     "he_attention_plain_workspace_floats": [c_int, c_int, c_int, c_int, c_int, c_int],
     "he_attention_plain": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int,
                            c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_ptr, c_int, c_ptr, c_i64,
-                           c_int, c_int, c_ptr, c_i64, c_ptr, c_ptr],
+                           c_int, c_int, c_ptr, c_i64, c_ptr, c_ptr, c_int, c_f32, c_ptr],
     "he_attention_decode_bf16": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int,
                                  c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_int, c_ptr,
-                                 c_i64, c_int, c_ptr, c_int, c_ptr, c_i64, c_ptr, c_ptr],
+                                 c_i64, c_int, c_ptr, c_int, c_ptr, c_i64, c_ptr, c_ptr, c_int, c_f32, c_ptr],
     "he_attention_decode_workspace_floats": [c_int, c_int, c_int, c_int, c_int],
     "he_attention_decode_fused_ok": [c_int, c_int, c_int, c_int],
     "he_attention_decode_fused_workspace_floats": [c_int, c_int, c_int, c_int, c_int, c_int],
@@ -106,7 +110,7 @@ _SIGNATURES = {
                                        c_int, c_int, c_f32, c_int, c_int, c_int, c_int, c_ptr, c_i64, c_ptr],
     "he_attention_prefill_bf16": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int,
                                   c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_int,
-                                  c_int, c_int, c_ptr, c_i64, c_int, c_ptr, c_int, c_ptr, c_i64, c_ptr, c_ptr],
+                                  c_int, c_int, c_ptr, c_i64, c_int, c_ptr, c_int, c_ptr, c_i64, c_ptr, c_ptr, c_int, c_f32, c_ptr],
     "he_attention_prefill_parts": [c_int, c_int, c_int, c_int, c_int],
     "he_attention_prefill_workspace_floats": [c_int, c_int, c_int, c_int],
     "he_argmax_workspace_bytes": [c_int, c_int],

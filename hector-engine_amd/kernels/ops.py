@@ -101,25 +101,29 @@ def gather_rows_f32(out, src, rows_idx, n_out: int, n_src: int) -> None:
 
 
 @_op("residual_add")
-def residual_add(resid_f32, delta, rows: int, scale: float = 1.0) -> None:
-    """resid += scale * delta."""
+def residual_add(resid_f32, delta, rows: int, scale: float = 1.0, delta2=None) -> None:
+    """resid += scale * (delta + delta2) (delta2 None: delta alone)."""
     D = resid_f32.shape[-1]
     _need(resid_f32, "resid", torch.float32)
     _need(delta, "delta")
     if delta.shape[-1] != D or resid_f32.numel() < rows * D or delta.numel() < rows * D:
         raise ValueError("residual_add: shape mismatch")
+    if delta2 is not None:
+        _need(delta2, "delta2", delta.dtype)
+        if delta2.shape[-1] != D or delta2.numel() < rows * D:
+            raise ValueError("residual_add: shape mismatch")
     L = _lib.load()
-    _lib.check(L.he_residual_add(resid_f32.data_ptr(), delta.data_ptr(), rows * D,
+    _lib.check(L.he_residual_add(resid_f32.data_ptr(), delta.data_ptr(), _ptr(delta2), rows * D,
                                  dtype_code(delta.dtype), float(scale), _stream()))
 
 
 @_op("silu_mul")
 def silu_mul(out, gate_up, rows: int, interleaved: bool = False, splits: int = 0, *,
-             alpha: float = 1.0, limit: float = 0.0, up_shift: float = 0.0) -> None:
+             alpha: float = 1.0, limit: float = 0.0, up_shift: float = 0.0, cubic: float = 0.0) -> None:
     """out[rows, I] = silu(gate) * up. gate_up: [rows, 2I] in out's dtype, or with
     splits > 0 the fp32 K slices [splits, rows, 2I] of the product. Its columns are all
     gates then all ups, or, interleaved, gate i in column 2i and its up in 2i + 1.
-    With constants it is the gated activation g' * sigmoid(alpha * g') * (u' + up_shift),
+    With constants it is the gated activation g' * sigmoid(alpha * g' + cubic * g'^3) * (u' + up_shift),
     g' = min(gate, limit), u' = clamp(up, -limit, limit) (limit 0: unbounded)."""
     I = out.shape[-1]
     _need(out, "out")
@@ -131,12 +135,12 @@ def silu_mul(out, gate_up, rows: int, interleaved: bool = False, splits: int = 0
         raise ValueError("silu_mul: split sums must be [splits, rows, 2*I]")
     L = _lib.load()
     _lib.check(L.he_gated_act(out.data_ptr(), gate_up.data_ptr(), rows, I, int(interleaved), splits,
-                              dtype_code(out.dtype), float(alpha), float(limit), float(up_shift), _stream()))
+                              dtype_code(out.dtype), float(alpha), float(limit), float(up_shift), float(cubic), _stream()))
 
 
 @_op("add_dyt")
-def add_dyt(resid_f32, delta, weight, bias, alpha, out, rows: int, delta_scale: float = 1.0) -> None:
-    """resid += delta_scale * delta (if given); out = tanh(alpha * resid) * weight + bias (if out given).
+def add_dyt(resid_f32, delta, weight, bias, alpha, out, rows: int, delta_scale: float = 1.0, delta2=None) -> None:
+    """resid += delta_scale * (delta + delta2) (if given, delta2 only with delta); out = tanh(alpha * resid) * weight + bias (if out given).
     alpha: a tensor of one element on the device; weight, bias: [D]; the three share a dtype."""
     D = resid_f32.shape[-1]
     _need(resid_f32, "resid", torch.float32)
@@ -160,8 +164,12 @@ def add_dyt(resid_f32, delta, weight, bias, alpha, out, rows: int, delta_scale: 
         if act is not None and delta.dtype != act:
             raise TypeError("add_dyt: delta and out must share a dtype")
         act = delta.dtype
+    if delta2 is not None:
+        _need(delta2, "delta2", act)
+        if delta is None or delta2.shape[-1] != D or delta2.numel() < rows * D:
+            raise ValueError(f"add_dyt: delta2 goes with delta and matches [rows, {D}]")
     L = _lib.load()
-    _lib.check(L.he_add_dyt(resid_f32.data_ptr(), _ptr(delta), float(delta_scale), weight.data_ptr(),
+    _lib.check(L.he_add_dyt(resid_f32.data_ptr(), _ptr(delta), _ptr(delta2), float(delta_scale), weight.data_ptr(),
                             bias.data_ptr(), alpha.data_ptr(), _ptr(out), rows, D,
                             dtype_code(act or torch.float32), dtype_code(weight.dtype), _stream()))
 
@@ -274,6 +282,11 @@ def gemm_blocksplit_blocks(M: int, N: int, K: int) -> int:
     return int(_lib.load().he_gemm_blocksplit_blocks(M, N, K))
 
 
+def _act4(act) -> tuple:
+    """(alpha, limit, up_shift, cubic) of a gated activation's constants, the last one 0 where it is left out."""
+    return tuple(float(a) for a in act) + (0.0,) * (4 - len(act))
+
+
 @_op("gemm_blocksplit")
 def gemm_blocksplit(out, a, w, bias, M: int, gated: bool = False, plan=(0, 0, 0), *,
                     row_scale=None, residual=None, x_pieces: bool = False, out_pieces: bool = False,
@@ -281,8 +294,8 @@ def gemm_blocksplit(out, a, w, bias, M: int, gated: bool = False, plan=(0, 0, 0)
     """bf16 MFMA product for M <= 32 with K cut inside the workgroup; one launch, complete
     result (bf16 or fp32), with bias or, gated, as [M, N/2] = silu(gate) * up for a weight
     that alternates gate and up rows (gate i at row 2i, its up at 2i + 1). plan = (R, U, NW),
-    zeros = heuristic. act = (alpha, limit, up_shift): the gated epilogue's constants as silu_mul
-    takes them.
+    zeros = heuristic. act = (alpha, limit, up_shift[, cubic]): the gated epilogue's
+    constants as silu_mul takes them.
 
     row_scale = (partials fp32 [M, count], eps): the rows of `a` are r * gain of an RMS norm
     whose 1/sqrt(mean(r^2) + eps) is applied to the sums here (mean over K).
@@ -350,7 +363,7 @@ def gemm_blocksplit(out, a, w, bias, M: int, gated: bool = False, plan=(0, 0, 0)
         dtype_code(out.dtype) if out is not None else BF16,
         dtype_code(bias.dtype) if bias is not None else F32, int(gated),
         int(plan[0]), int(plan[1]), int(plan[2]), sp, sc, float(se), rp, gp, gdt, xp, qp, qc,
-        int(x_pieces), int(out_pieces), float(act[0]), float(act[1]), float(act[2]), float(rscale),
+        int(x_pieces), int(out_pieces), *_act4(act), float(rscale),
         _ptr(dyt_bias), _ptr(dyt_alpha), _stream()))
 
 
@@ -429,7 +442,7 @@ def gemm_rows(out, partial, a, w, bias, M: int, gated: bool = False, plan=(0, 0,
         dtype_code(out.dtype) if out is not None else BF16,
         dtype_code(bias.dtype) if bias is not None else F32, int(gated),
         int(plan[0]), int(plan[1]), int(plan[2]), sp, sc, float(se), rp, gp, gdt, xp, qp, qc,
-        int(x_pieces), int(out_pieces), ctypes.byref(used), float(act[0]), float(act[1]), float(act[2]),
+        int(x_pieces), int(out_pieces), ctypes.byref(used), *_act4(act),
         float(rscale), _ptr(dyt_bias), _ptr(dyt_alpha), _stream()))
     return used.value
 
@@ -792,33 +805,72 @@ def gated_add(out, a, b, x, gate_weight, rows: int) -> None:
 
 
 @_op("head_product")
-def head_product(out, x, w, rows: int) -> None:
+def head_product(out, x, w, rows: int, gate=None, transposed: bool = False) -> None:
     """out[r, h, :] = x[r, h, :] @ w[h] for views out [rows, H, N] and x [rows, H, K] (unit stride along the last
-    axis, any row and head strides) and w [H, K, N]; fp32 sums in ascending k."""
-    H, K, N = w.shape
-    _need(w, "w")
+    axis, any row and head strides) and w [H, K, N]; fp32 sums in ascending k. gate (a view [rows, H * N] of wider
+    rows in x's dtype): the result is multiplied by sigmoid(gate). transposed: w is [H, N, K] and the product runs on
+    the matrix cores (bf16; what head_product_mfma_ok asks of the sizes)."""
+    H, K, N = (w.shape[0], w.shape[2], w.shape[1]) if transposed else w.shape
+    _need(w, "w", torch.bfloat16 if transposed else None)
     for name, t, last in (("x", x, K), ("out", out, N)):
         if not t.is_cuda or t.dtype != x.dtype or t.dim() != 3 or t.shape[1] != H or t.shape[2] != last \
                 or t.stride(2) != 1 or t.shape[0] < rows:
             raise ValueError(f"head_product: {name} must be a [rows, {H}, {last}] view with unit stride along the last axis")
+    if gate is not None and (not gate.is_cuda or gate.dtype != x.dtype or gate.dim() != 2 or gate.shape[1] != H * N
+                             or gate.stride(1) != 1 or gate.shape[0] < rows):
+        raise ValueError(f"head_product: gate must be a [rows, {H * N}] view in x's dtype")
+    gp, gr = (None, 0) if gate is None else (gate.data_ptr(), gate.stride(0))
     L = _lib.load()
+    if transposed:
+        if x.dtype != torch.bfloat16:
+            raise TypeError("head_product: the matrix cores take bfloat16 rows")
+        _lib.check(L.he_head_product_mfma(out.data_ptr(), out.stride(0), out.stride(1), x.data_ptr(), x.stride(0), x.stride(1),
+                                          w.data_ptr(), rows, H, K, N, gp, gr, _stream()))
+        return
     _lib.check(L.he_head_product(out.data_ptr(), out.stride(0), out.stride(1), x.data_ptr(), x.stride(0), x.stride(1),
-                                 w.data_ptr(), dtype_code(w.dtype), rows, H, K, N, dtype_code(x.dtype), _stream()))
+                                 w.data_ptr(), dtype_code(w.dtype), rows, H, K, N, gp, gr, dtype_code(x.dtype), _stream()))
 
 
-@_op("latent_pack")
-def latent_pack(qkv, q, down, rows: int, H: int, d: int, r: int, rank: int) -> None:
-    """qkv [rows, H (r + rank) + (r + rank) + rank]: head h's first r columns = the last r of q[row, h] (q [rows, H (d + r)]),
-    the key = [down[row, rank:rank + r] | down[row, :rank]], the value = down[row, :rank] (down: a view [rows, rank + r])."""
-    hd = r + rank
-    _need(qkv, "qkv", None, (None, (H + 1) * hd + rank))
-    _need(q, "q", qkv.dtype, (None, H * (d + r)))
-    if not down.is_cuda or down.dtype != qkv.dtype or down.dim() != 2 or down.shape[1] != rank + r or down.stride(1) != 1 \
-            or min(down.shape[0], q.shape[0], qkv.shape[0]) < rows:
-        raise ValueError("latent_pack: down must be a [rows, rank + r] view in qkv's dtype")
+def head_product_mfma_ok(K: int, x_row: int, x_head: int) -> bool:
+    """Whether head_product's matrix-core form takes this inner size and these strides of x (elements)."""
+    return K % 8 == 0 and x_row % 8 == 0 and x_head % 8 == 0
+
+
+@_op("latent_cache")
+def latent_cache(q_out, kpool, vpool, q, down, gain, eps: float, positions, row_seq, seq_slot, page_table, inv_freq, rows: int,
+                 H: int, d: int, r: int, rank: int, pd: int, *, interleaved: bool = False, mscale: float = 1.0) -> None:
+    """The projected rows of a latent attention's step, one launch. q (a view [rows, H (d + r)]): a head's last r dims,
+    rotated at the row's position, go to the first r dims of its pd dims of q_out [rows, H pd], zeros behind its first
+    r + rank; the dims r .. r + rank are left to the head product that follows or precedes. down (a view [rows, rank + r],
+    or None: the latents are another run's): c = rms(down[:, :rank]) * gain; the key [rotated down[:, rank:] | c] and the
+    value c go into the pools (one kv head of pd dims) at (slot, position)."""
+    _need(q_out, "q_out", None, (None, H * pd))
+    for name, t, cols in (("q", q, H * (d + r)), ("down", down, rank + r)):
+        if t is not None and (not t.is_cuda or t.dtype != q_out.dtype or t.dim() != 2 or t.shape[1] != cols or t.stride(1) != 1
+                              or t.shape[0] < rows):
+            raise ValueError(f"latent_cache: {name} must be a [rows, {cols}] view in q_out's dtype")
+    if q_out.shape[0] < rows:
+        raise ValueError("latent_cache: q_out has fewer rows than the step")
+    for name, t in (("positions", positions), ("row_seq", row_seq), ("seq_slot", seq_slot)):
+        _need(t, name, torch.int32)
+    if positions.numel() < rows or row_seq.numel() < rows:
+        raise ValueError("latent_cache: metadata shorter than the row count")
+    if r:
+        _need(inv_freq, "inv_freq", torch.float32, (r // 2,))
+    max_blocks = num_pages = 0
+    if down is not None:
+        _need(gain, "gain", None, (rank,))
+        _need(kpool, "kpool", q_out.dtype, (None, 1, layout.k_page_elems(pd)))
+        _need(vpool, "vpool", q_out.dtype, (None, 1, layout.v_page_elems(pd)))
+        _need(page_table, "page_table", torch.int32)
+        num_pages, max_blocks = kpool.shape[0], page_table.shape[1]
     L = _lib.load()
-    _lib.check(L.he_latent_pack(qkv.data_ptr(), q.data_ptr(), down.data_ptr(), down.stride(0), rows, H, d, r, rank,
-                                dtype_code(qkv.dtype), _stream()))
+    _lib.check(L.he_latent_cache(
+        q_out.data_ptr(), q_out.stride(0), _ptr(kpool) if down is not None else None, _ptr(vpool) if down is not None else None,
+        q.data_ptr(), q.stride(0), _ptr(down), down.stride(0) if down is not None else 0, _ptr(gain) if down is not None else None,
+        dtype_code(gain.dtype) if down is not None else F32, float(eps), positions.data_ptr(), row_seq.data_ptr(),
+        seq_slot.data_ptr(), _ptr(page_table) if down is not None else None, max_blocks, num_pages, _ptr(inv_freq) if r else None,
+        int(interleaved), float(mscale), rows, H, d, r, rank, pd, dtype_code(q_out.dtype), _stream()))
 
 
 @_op("add_normed")
@@ -959,33 +1011,42 @@ def mlstm_scan(y, q, k, v, gates, state, state_offset: int, cu_seqlens, seq_slot
 
 @_op("route_tokens")
 def route_tokens(dense, ids, weights, logits, correction, rows: int, real: int, groups: int, keep: int,
-                 top: int, scale: float, *, x=None, router=None, normalize: bool = False) -> None:
+                 top: int, scale: float, *, x=None, router=None, normalize: bool = False, bias=None,
+                 x_pieces: bool = False) -> None:
     """The choice of `top` of E router outputs per row (logits fp32 [rows, E]; or logits None and the kernel
     forms them in fp32 from the rows x [rows, D] and the router's matrix, fp32 [E, D]): softmax scores s, the
     choice on s + correction inside the `keep` best of `groups` equal groups, weights s * scale. dense (fp32
     [rows, real + 1]): each expert's weight or 0, the outputs from `real` on added up in the last column;
     ids (int32) and weights (fp32) [rows, top]: the chosen outputs. normalize: the chosen outputs' weights are divided
-    by their sum (times scale): the softmax over the chosen logits alone."""
+    by their sum (times scale): the softmax over the chosen logits alone. bias [E]: added to the logits first.
+    x_pieces: x lies piece-major, shaped pieces_shape(rows, D)."""
     if logits is None:
         E, D = router.shape
         _need(router, "router", torch.float32)
-        _need(x, "x", None, (None, D))
-        if x.shape[0] < rows:
-            raise ValueError("route_tokens: x has fewer rows than the step")
-        return _route(dense, ids, weights, None, x, router, correction, rows, E, real, groups, keep, top, scale, normalize)
+        if x_pieces:
+            _need(x, "x", torch.bfloat16, pieces_shape(rows, D))
+        else:
+            _need(x, "x", None, (None, D))
+            if x.shape[0] < rows:
+                raise ValueError("route_tokens: x has fewer rows than the step")
+        return _route(dense, ids, weights, None, x, router, correction, rows, E, real, groups, keep, top, scale, normalize,
+                      bias, x_pieces)
     E = logits.shape[-1]
     _need(logits, "logits", torch.float32, (None, E))
     if logits.shape[0] < rows:
         raise ValueError("route_tokens: buffers smaller than the row count")
-    _route(dense, ids, weights, logits, None, None, correction, rows, E, real, groups, keep, top, scale, normalize)
+    _route(dense, ids, weights, logits, None, None, correction, rows, E, real, groups, keep, top, scale, normalize, bias)
 
 
-def _route(dense, ids, weights, logits, x, router, correction, rows, E, real, groups, keep, top, scale, normalize=False) -> None:
+def _route(dense, ids, weights, logits, x, router, correction, rows, E, real, groups, keep, top, scale, normalize=False,
+           bias=None, x_pieces=False) -> None:
     _need(dense, "dense", torch.float32, (None, real + 1))
     _need(ids, "ids", torch.int32, (None, top))
     _need(weights, "weights", torch.float32, (None, top))
     if correction is not None:
         _need(correction, "correction", None, (E,))
+    if bias is not None:
+        _need(bias, "bias", None, (E,))
     if min(dense.shape[0], ids.shape[0], weights.shape[0]) < rows:
         raise ValueError("route_tokens: buffers smaller than the row count")
     L = _lib.load()
@@ -993,18 +1054,19 @@ def _route(dense, ids, weights, logits, x, router, correction, rows, E, real, gr
                                  _ptr(x), dtype_code(x.dtype) if x is not None else F32, _ptr(router),
                                  router.shape[1] if router is not None else 0,
                                  _ptr(correction), dtype_code(correction.dtype) if correction is not None else F32,
-                                 rows, E, real, groups, keep, top, float(scale), int(normalize), _stream()))
+                                 rows, E, real, groups, keep, top, float(scale), int(normalize), _ptr(bias),
+                                 dtype_code(bias.dtype) if bias is not None else F32, int(x_pieces), _stream()))
 
 
 @_op("routed_act")
-def routed_act(out, gate_up, dense, h, rows: int, real: int, inter: int, *, alpha: float = 1.0,
-               limit: float = 0.0, up_shift: float = 0.0) -> None:
-    """out[rows, real * inter + extra]: the experts' gated activations (gate_up [rows, 2 real inter], gate and
-    up alternating) times their weights dense[row, e]; the last extra = h.shape[1] columns (h None: none)
-    are dense[row, real] * h."""
+def routed_act(out, gate_up, dense, h, rows: int, real: int, inter: int, *, shared: int = 0, alpha: float = 1.0,
+               limit: float = 0.0, up_shift: float = 0.0, cubic: float = 0.0) -> None:
+    """out[rows, real * inter + shared + extra]: the experts' gated activations (gate_up [rows, 2 (real inter +
+    shared)], gate and up alternating) times their weights dense[row, e], the `shared` columns with weight 1; the
+    last extra = h.shape[1] columns (h None: none) are dense[row, real] * h."""
     extra = 0 if h is None else h.shape[1]
-    _need(out, "out", None, (None, real * inter + extra))
-    _need(gate_up, "gate_up", out.dtype, (None, 2 * real * inter))
+    _need(out, "out", None, (None, real * inter + shared + extra))
+    _need(gate_up, "gate_up", out.dtype, (None, 2 * (real * inter + shared)))
     _need(dense, "dense", torch.float32, (None, real + 1))
     if h is not None:
         _need(h, "h", out.dtype)
@@ -1012,32 +1074,42 @@ def routed_act(out, gate_up, dense, h, rows: int, real: int, inter: int, *, alph
         raise ValueError("routed_act: buffers smaller than the row count")
     L = _lib.load()
     _lib.check(L.he_routed_act(out.data_ptr(), gate_up.data_ptr(), dense.data_ptr(), _ptr(h), rows, real, inter,
-                               extra, dtype_code(out.dtype), float(alpha), float(limit), float(up_shift), _stream()))
+                               shared, extra, dtype_code(out.dtype), float(alpha), float(limit), float(up_shift), float(cubic),
+                               _stream()))
 
 
 @_op("chosen_experts")
 def chosen_experts(out, h_scratch, x, gate_up, down, ids, weights, dense, rows: int, real: int, inter: int, *,
-                   alpha: float = 1.0, limit: float = 0.0, up_shift: float = 0.0) -> None:
+                   shared: int = 0, x_pieces: bool = False, alpha: float = 1.0, limit: float = 0.0, up_shift: float = 0.0,
+                   cubic: float = 0.0) -> None:
     """For a step of very few bf16 rows: out[rows, D] = the weighted sum of the chosen experts' results alone
     (ids, weights [rows, top] and dense [rows, real + 1] as route_tokens leaves them), read from the fused matrices
-    of the products over all experts: gate_up [2 real inter, D] (gate and up alternating), down [D, real inter (+ D)].
-    The identity experts' share dense[row, real] * x is added. h_scratch: bf16 [rows * top, inter]."""
-    D = x.shape[1]
+    of the products over all experts: gate_up [2 (real inter + shared), D] (gate and up alternating), down
+    [D, real inter + shared (+ D)]; the `shared` columns belong to an expert every row uses with weight 1.
+    The identity experts' share dense[row, real] * x is added. h_scratch: bf16, rows * (top * inter + shared) elements.
+    x_pieces: x lies piece-major (no identity experts then)."""
+    D = gate_up.shape[1]
     top = ids.shape[1]
     for name, t in (("out", out), ("h_scratch", h_scratch), ("x", x), ("gate_up", gate_up), ("down", down)):
         _need(t, name, torch.bfloat16)
     _need(ids, "ids", torch.int32, (None, top))
     _need(weights, "weights", torch.float32, (None, top))
     _need(dense, "dense", torch.float32, (None, real + 1))
-    if tuple(gate_up.shape) != (2 * real * inter, D) or down.shape[0] != D or down.shape[1] < real * inter:
+    if tuple(gate_up.shape) != (2 * (real * inter + shared), D) or down.shape[0] != D \
+            or down.shape[1] not in (real * inter + shared, real * inter + shared + D):
         raise ValueError("chosen_experts: the fused matrices do not match the sizes")
-    if min(out.shape[0], x.shape[0], ids.shape[0], weights.shape[0], dense.shape[0]) < rows or out.shape[1] != D \
-            or h_scratch.numel() < rows * top * inter:
+    if x_pieces:
+        _need(x, "x", shape=pieces_shape(rows, D))
+    elif x.shape[0] < rows or x.shape[1] != D:
+        raise ValueError("chosen_experts: x must be [rows, D]")
+    if min(out.shape[0], ids.shape[0], weights.shape[0], dense.shape[0]) < rows or out.shape[1] != D \
+            or h_scratch.numel() < rows * (top * inter + shared):
         raise ValueError("chosen_experts: buffers smaller than the row count")
     L = _lib.load()
     _lib.check(L.he_chosen_experts(out.data_ptr(), h_scratch.data_ptr(), x.data_ptr(), gate_up.data_ptr(), down.data_ptr(),
                                    down.stride(0), ids.data_ptr(), weights.data_ptr(), dense.data_ptr(), rows, top, real,
-                                   inter, D, float(alpha), float(limit), float(up_shift), _stream()))
+                                   inter, shared, D, float(alpha), float(limit), float(up_shift), float(cubic), int(x_pieces),
+                                   _stream()))
 
 
 @_op("diff_heads")
@@ -1068,7 +1140,8 @@ def _check_attention(out, q, kpool, vpool, page_table, rows, H, KVH, hd):
 @_op("attention_plain")
 def attention_plain(out, q, kpool, vpool, positions, row_seq, seq_slot, page_table, rows: int,
                     H: int, KVH: int, hd: int, window: int, scale: float, most_keys: int = 0,
-                    workspace=None, *, chunk: int = 0, sinks=None, gate=None, slopes=None) -> None:
+                    workspace=None, *, chunk: int = 0, sinks=None, gate=None, slopes=None, cap: float = 0.0,
+                    table=None) -> None:
     """most_keys: a bound on the keys any sequence holds after the step, and workspace: fp32, of
     attention_plain_workspace_floats elements or more: the pages of a query then run in parallel
     (a step of few queries over many keys); the result is the same bit for bit without them.
@@ -1076,13 +1149,13 @@ def attention_plain(out, q, kpool, vpool, positions, row_seq, seq_slot, page_tab
     position 0). sinks [H]: a number a head that joins the softmax's denominator as exp(sink).
     gate: a view [rows, H] of q's dtype (unit stride along heads, any row stride): the head's output
     is multiplied by sigmoid(gate). slopes (fp32 [H]): the score of key j for the query at p loses
-    slopes[h] * (p - j)."""
+    slopes[h] * (p - j). cap > 0: a score s becomes cap * tanh(s / cap). table (fp32 [H, entries]): the score then
+    gains table[h, min(p - j, entries - 1)] (not together with slopes)."""
     _check_attention(out, q, kpool, vpool, page_table, rows, H, KVH, hd)
     gate_ptr, gate_stride = _gate_view(gate, q, rows, H)
     if sinks is not None:
         _need(sinks, "sinks", shape=(H,))
-    if slopes is not None:
-        _need(slopes, "slopes", torch.float32, (H,))
+    _check_shape(slopes, cap, table, H)
     if workspace is not None:
         _need(workspace, "workspace", torch.float32)
     for name, t in (("positions", positions), ("row_seq", row_seq), ("seq_slot", seq_slot)):
@@ -1096,7 +1169,26 @@ def attention_plain(out, q, kpool, vpool, positions, row_seq, seq_slot, page_tab
         kpool.shape[0], rows, H, KVH, hd, window, int(chunk), float(scale), _ptr(sinks),
         dtype_code(sinks.dtype) if sinks is not None else F32, gate_ptr, gate_stride,
         dtype_code(q.dtype), int(most_keys),
-        _ptr(workspace), workspace.numel() if workspace is not None else 0, _ptr(slopes), _stream()))
+        _ptr(workspace), workspace.numel() if workspace is not None else 0, _ptr(slopes), *_table_args(table, cap), _stream()))
+
+
+# the longest distance table the prompt kernel that shares pages through LDS takes
+ATTENTION_TABLE_LDS = 2048
+
+
+def _check_shape(slopes, cap: float, table, H: int) -> None:
+    if slopes is not None:
+        _need(slopes, "slopes", torch.float32, (H,))
+        if cap > 0 or table is not None:
+            raise ValueError("attention: slopes go with neither a cap nor a distance table")
+    if table is not None:
+        _need(table, "table", torch.float32, (H, None))
+    if cap < 0:
+        raise ValueError("attention: the score cap must not be negative")
+
+
+def _table_args(table, cap: float):
+    return _ptr(table), table.shape[1] if table is not None else 0, float(cap)
 
 
 def _gate_view(gate, q, rows: int, H: int):
@@ -1121,15 +1213,15 @@ def attention_decode_workspace_floats(rows: int, H: int, KVH: int, hd: int, max_
 @_op("attention_decode")
 def attention_decode(out, q, kpool, vpool, positions, row_seq, seq_slot, page_table, rows: int,
                      H: int, KVH: int, hd: int, window: int, scale: float, max_keys: int,
-                     workspace, *, chunk: int = 0, sinks=None, gate=None, slopes=None) -> None:
-    """chunk, sinks, gate, slopes: as attention_plain takes them."""
+                     workspace, *, chunk: int = 0, sinks=None, gate=None, slopes=None, cap: float = 0.0,
+                     table=None) -> None:
+    """chunk, sinks, gate, slopes, cap, table: as attention_plain takes them."""
     _check_attention(out, q, kpool, vpool, page_table, rows, H, KVH, hd)
     _need(q, "q", torch.bfloat16)
     gate_ptr, gate_stride = _gate_view(gate, q, rows, H)
     if sinks is not None:
         _need(sinks, "sinks", shape=(H,))
-    if slopes is not None:
-        _need(slopes, "slopes", torch.float32, (H,))
+    _check_shape(slopes, cap, table, H)
     for name, t in (("positions", positions), ("row_seq", row_seq), ("seq_slot", seq_slot)):
         _need(t, name, torch.int32)
     if positions.numel() < rows or row_seq.numel() < rows:
@@ -1141,7 +1233,7 @@ def attention_decode(out, q, kpool, vpool, positions, row_seq, seq_slot, page_ta
         row_seq.data_ptr(), seq_slot.data_ptr(), page_table.data_ptr(), page_table.shape[1],
         kpool.shape[0], rows, H, KVH, hd, window, float(scale), max_keys, workspace.data_ptr(),
         workspace.numel(), int(chunk), _ptr(sinks), dtype_code(sinks.dtype) if sinks is not None else F32,
-        gate_ptr, gate_stride, _ptr(slopes), _stream()))
+        gate_ptr, gate_stride, _ptr(slopes), *_table_args(table, cap), _stream()))
 
 
 def attention_decode_fused_ok(H: int, KVH: int, hd: int, rotary_dim: int) -> bool:
@@ -1224,19 +1316,19 @@ def attention_prefill_workspace_floats(total_rows: int, H: int, hd: int, parts: 
 def attention_prefill(out, q, kpool, vpool, cu_seqlens, seq_slot, seq_start, page_table,
                       num_seqs: int, max_q_len: int, total_rows: int, H: int, KVH: int, hd: int,
                       window: int, scale: float, kernel: int = 0, parts: int = 1, workspace=None, *,
-                      chunk: int = 0, sinks=None, gate=None, slopes=None) -> None:
+                      chunk: int = 0, sinks=None, gate=None, slopes=None, cap: float = 0.0, table=None) -> None:
     """kernel: 0 leaves the choice to the library (by head size and prompt length); 1 or 2
     name it: 16 queries a wavefront with operands from global memory, or 32 queries a
     wavefront with the pages shared through LDS (head sizes up to 128). parts > 1 (kernel 2):
     the keys in that many parts side by side, joined by a second launch; the workspace holds
-    attention_prefill_workspace_floats() floats. chunk, sinks, gate, slopes: as attention_plain takes them."""
+    attention_prefill_workspace_floats() floats. chunk, sinks, gate, slopes, cap, table: as attention_plain takes them
+    (kernel 2: tables of up to ATTENTION_TABLE_LDS entries)."""
     _check_attention(out, q, kpool, vpool, page_table, total_rows, H, KVH, hd)
     _need(q, "q", torch.bfloat16)
     gate_ptr, gate_stride = _gate_view(gate, q, total_rows, H)
     if sinks is not None:
         _need(sinks, "sinks", shape=(H,))
-    if slopes is not None:
-        _need(slopes, "slopes", torch.float32, (H,))
+    _check_shape(slopes, cap, table, H)
     for name, t in (("cu_seqlens", cu_seqlens), ("seq_slot", seq_slot), ("seq_start", seq_start)):
         _need(t, name, torch.int32)
     if cu_seqlens.numel() < num_seqs + 1 or seq_slot.numel() < num_seqs or seq_start.numel() < num_seqs:
@@ -1250,7 +1342,7 @@ def attention_prefill(out, q, kpool, vpool, cu_seqlens, seq_slot, seq_start, pag
         kpool.shape[0], num_seqs, max_q_len, H, KVH, hd, window, float(scale), int(kernel),
         total_rows, int(parts), _ptr(workspace), workspace.numel() if workspace is not None else 0,
         int(chunk), _ptr(sinks), dtype_code(sinks.dtype) if sinks is not None else F32, gate_ptr, gate_stride,
-        _ptr(slopes), _stream()))
+        _ptr(slopes), *_table_args(table, cap), _stream()))
 
 
 @_op("argmax_rows")

@@ -38,6 +38,11 @@ Options of the same part, each off unless its parameter says otherwise:
               the q/k norm (behind the convolution). value_dim must equal head_dim.
   distance_slope_span  s > 0: the score of key j for the query at position i loses slope_h * (i - j), with
               slope_h = 2^(-s (h + 1) / H) for head h.
+  score_cap   c > 0: a score s (q . k * scale) becomes c * tanh(s / c).
+  distance_table  {far: D} (rows: the B of a random model): a stored table `distance` [B, H]; the (capped) score of key j for the query at
+              position i gains row bucket(i - j) of it. Of the B rows the first floor(B/2) =: F are the distances
+              0 .. F - 1; distance n >= F has the row F + floor(ln(n / F) / ln(D / F) * (B - F)), at most B - 1
+              (distance_bucket). The kernels read it spread out over the distances.
   q_temp      {coef, every}: the q of position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).
   score_maps  2: differential attention. A head has two queries and a kv head two keys (in the q and k
               matrices a head's rows for map 1 stand in front of its rows for map 2); the two maps are
@@ -48,7 +53,7 @@ Options of the same part, each off unless its parameter says otherwise:
               so that the heads of one (kv head, map) are neighbours, and the value rows of a kv head
               stand once for each of its maps; ops.diff_heads then joins the pairs.
   names       the suffixes of its tensors (q, k, v, o, q_bias, k_bias, v_bias, o_bias, sinks, gate,
-              lq1, lk1, lq2, lk2, q_norm, k_norm, q_conv, k_conv).
+              lq1, lk1, lq2, lk2, q_norm, k_norm, q_conv, k_conv, distance).
 """
 from __future__ import annotations
 
@@ -64,7 +69,8 @@ from .base import (BuildEnv, KVNeed, LayerCache, Mixer, PartSpec, PieceRows, Ste
 _NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
           "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
           "sinks": "sinks", "gate": "gate.weight", "lq1": "lambda_q1", "lk1": "lambda_k1", "lq2": "lambda_q2",
-          "lk2": "lambda_k2", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "q_conv": "q_conv.weight", "k_conv": "k_conv.weight"}
+          "lk2": "lambda_k2", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "q_conv": "q_conv.weight", "k_conv": "k_conv.weight",
+          "distance": "distance_bias"}
 from .linear import Linear
 
 
@@ -84,6 +90,21 @@ def keys_uneven(lengths: list[int], before=None) -> bool:
     that a batch at the edge does not go back and forth between two graphs."""
     longest = max(lengths)
     return longest >= 4096 and longest * len(lengths) >= (3 if before else 4) * sum(lengths)
+
+
+def distance_bucket(n: int, rows: int, far: int) -> int:
+    """The row of a distance table of `rows` rows for a key n >= 0 positions back (see distance_table above). The
+    logarithms are compared exactly: floor(m ln(n / F) / ln(far / F)) >= k is n^m F^k >= far^k F^m in integers."""
+    first = rows // 2
+    if n < first:
+        return n
+    if first == 0 or far <= first:
+        return rows - 1
+    m = rows - first
+    k = 0
+    while k < m - 1 and n ** m * first ** (k + 1) >= far ** (k + 1) * first ** m:
+        k += 1
+    return first + k
 
 
 @register_part("mixer", "attention")
@@ -115,6 +136,10 @@ class Attention(Mixer):
         self.values_are_keys = param(params, "values", str, "projection") == "keys"
         self.slope_span = param(params, "distance_slope_span", float, 0.0)
         self.slopes: torch.Tensor | None = None
+        self.score_cap = param(params, "score_cap", float, 0.0)
+        dt = param(params, "distance_table", dict, None)
+        self.table_rows, self.table_far = (int(dt.get("rows", 32)), int(dt["far"])) if dt else (0, 0)
+        self.table: torch.Tensor | None = None      # fp32 [H, distances]: the stored table spread out (bind)
         self.taps = None
         self.maps = param(params, "score_maps", int, 1)
         self.diff = param(params, "diff", float, 0.0)
@@ -137,6 +162,10 @@ class Attention(Mixer):
             raise ValueError("attention: conv_taps and values 'keys' go without biases, gates, score maps and shared caches")
         if self.values_are_keys and self.vd != self.hd:
             raise ValueError(f"attention: values that are the keys are head_dim {self.hd} wide, not {self.vd}")
+        if self.score_cap < 0 or (dt and min(self.table_rows, self.table_far) < 1):
+            raise ValueError("attention: score_cap must not be negative, rows and far of a distance_table must be positive")
+        if (self.score_cap or dt) and (self.slope_span or self.maps > 1):
+            raise ValueError("attention: score_cap and distance_table go without distance slopes and score maps")
         if self.has_sinks and self.sink_value is not None:
             raise ValueError("attention: stored sinks and sink_value exclude each other")
         if self.q_temp is not None and self.q_temp[1] <= 0:
@@ -166,7 +195,7 @@ class Attention(Mixer):
         # what the fused one-token kernel and the kernels without these options do not take
         self.extras = self.chunk > 0 or self.has_sinks or self.head_gate or self.maps > 1 or self.q_temp is not None \
             or self.out_gate or self.sink_value is not None or bool(self.qk_norm) or self.conv_taps > 0 \
-            or self.values_are_keys or self.slope_span > 0
+            or self.values_are_keys or self.slope_span > 0 or self.score_cap > 0 or self.table_rows > 0
         # rows of the gate's matrix behind q||k||v: one a head, or one for every value of every head
         self.gate_rows = self.H if self.head_gate else self.H * self.vd if self.out_gate else 0
 
@@ -205,6 +234,8 @@ class Attention(Mixer):
             specs[n["o_bias"]] = TensorSpec((self.hidden,))
         if self.has_sinks:
             specs[n["sinks"]] = TensorSpec((self.H,), ("normal", 1.0))
+        if self.table_rows:
+            specs[n["distance"]] = TensorSpec((None, self.H), ("normal", 1.0), free=self.table_rows)
         if self.gate_rows:
             specs[n["gate"]] = TensorSpec((self.gate_rows, self.hidden))
         if self.qk_norm:
@@ -274,6 +305,15 @@ class Attention(Mixer):
         if self.slope_span:
             h = torch.arange(1, self.H + 1, dtype=torch.float64)
             self.slopes = torch.exp2(-self.slope_span * h / self.H).to(torch.float32).to(wo.device)
+        if self.table_rows:
+            # beyond `far` (and the first half) nothing changes, and nothing beyond the window is seen: the kernels
+            # repeat the last entry
+            reach = max(self.table_far, tensors[n["distance"]].shape[0] // 2) + 1
+            reach = min(reach, self.window or reach)
+            stored = tensors[n["distance"]]
+            rows = torch.tensor([distance_bucket(x, stored.shape[0], self.table_far) for x in range(reach)],
+                                device=wo.device)
+            self.table = stored.float()[rows].t().contiguous()
         self.position.bind(tensors)
 
     def _by_map(self, which: str, t: torch.Tensor) -> torch.Tensor:
@@ -425,7 +465,7 @@ class Attention(Mixer):
         ops.attention_plain(out, q, cache.kpool, cache.vpool, ctx.positions, ctx.row_seq,
                             ctx.seq_slot, cache.page_table, rows, H, KVH, hd, self.window,
                             self.scale, ctx.most_keys, ws, chunk=self.chunk, sinks=self.sinks,
-                            gate=gate if self.head_gate else None, slopes=self.slopes)
+                            gate=gate if self.head_gate else None, slopes=self.slopes, cap=self.score_cap, table=self.table)
         return self._project(out, rows, ctx, gate)
 
     def _run_mfma_one_token(self, x, ctx: StepContext, cache: LayerCache):
@@ -438,7 +478,8 @@ class Attention(Mixer):
         ops.attention_decode(out, q, cache.kpool, cache.vpool, ctx.positions, ctx.row_seq,
                              ctx.seq_slot, cache.page_table, rows, H, KVH, hd, self.window,
                              self.scale, ctx.max_keys, ws, chunk=self.chunk, sinks=self.sinks,
-                             gate=gate if self.head_gate else None, slopes=self.slopes)
+                             gate=gate if self.head_gate else None, slopes=self.slopes, cap=self.score_cap,
+                             table=self.table)
         return self._project(out, rows, ctx, gate)
 
     def _run_mfma_prompt(self, x, ctx: StepContext, cache: LayerCache):
@@ -453,6 +494,8 @@ class Attention(Mixer):
         if self.chunk > 0:
             most = min(most, self.chunk + ctx.max_q_len)
         parts = ops.attention_prefill_parts(ctx.num_seqs, ctx.max_q_len, H, hd, most)
+        if self.table is not None and self.table.shape[1] > ops.ATTENTION_TABLE_LDS:
+            parts = 1                     # the kernel that cuts the keys keeps the head's table in LDS
         ws = ctx.alloc((ops.attention_prefill_workspace_floats(rows, H, hd, parts),), torch.float32) \
             if parts > 1 else None
         if ctx.padded:
@@ -463,7 +506,7 @@ class Attention(Mixer):
                               ctx.seq_start, cache.page_table, ctx.num_seqs, ctx.max_q_len,
                               rows, H, KVH, hd, self.window, self.scale, parts=parts, workspace=ws,
                               chunk=self.chunk, sinks=self.sinks, gate=gate if self.head_gate else None,
-                              slopes=self.slopes)
+                              slopes=self.slopes, cap=self.score_cap, table=self.table)
         return self._project(out, rows, ctx, gate)
 
 

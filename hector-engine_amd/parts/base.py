@@ -35,11 +35,20 @@ class TensorSpec:
     init: ("normal", std) | ("gain", mean, std) | ("zeros",) | ("constant", value), or any kind
     registered with weights.random_init.register_init
     integer: integer tables are kept as int32, everything else follows the run dtype rule.
+    free: a dim of None in `shape` is whatever the file stores (the part reads it from the tensor it is
+    bound to); a random model gets `free` there.
     """
 
     shape: tuple
     init: tuple = ("normal", 0.02)
     integer: bool = False
+    free: int = 1
+
+    def matches(self, stored) -> bool:
+        return len(stored) == len(self.shape) and all(a is None or a == b for a, b in zip(self.shape, stored))
+
+    def random_shape(self) -> tuple:
+        return tuple(self.free if a is None else a for a in self.shape)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -224,6 +233,9 @@ class Part:
 
 
 class Norm(Part):
+    # True for a norm whose add_norm takes a second branch output (delta2, added to delta)
+    takes_pair = False
+
     def carried(self) -> tuple | None:
         """(gain [D], eps) when the norm is y = x * gain / sqrt(mean(x^2) + eps), so that a
         pair of products can carry it (ResidualSink, NormedRows); (gain [D], 1.0, bias [D], alpha)
@@ -318,7 +330,7 @@ class NormedRows:
     """Rows of an RMS norm whose per-row scale is still owed: `scaled` = r * gain in the
     activation dtype, and the sum of r^2 of a row as `partials[row, :]` (fp32, added in
     index order by lanes of 64, then across the lanes). norm(r) = scaled / sqrt(sum / dim +
-    eps). A product applies the scale to its sums (parts.linear.Linear); tensor() gives the
+    eps). finished: nothing is owed, `scaled` holds the norm's rows themselves. A product applies the scale to its sums (parts.linear.Linear); tensor() gives the
     normalised rows to anything else. pieces: `scaled` lies piece-major
     (kernels.ops.pieces_shape(rows, dim))."""
 
@@ -327,6 +339,7 @@ class NormedRows:
     eps: float
     rows: int
     pieces: bool = False
+    finished: bool = False
 
     @property
     def dim(self) -> int:
@@ -368,7 +381,8 @@ class ResidualStream:
         self.resid = resid
         self.rows = rows
         self.pending: torch.Tensor | None = None
-        self.pending_scale = 1.0                               # the stream gains pending_scale * pending
+        self.pending2: torch.Tensor | None = None              # a second branch's, added with the first (add_pair)
+        self.pending_scale = 1.0                               # the stream gains pending_scale * (pending + pending2)
         self.prepared: tuple[Norm, NormedRows] | None = None   # rows already made for that norm
         self.ready: tuple[Norm, torch.Tensor] | None = None    # that norm of the stream as it stands, already computed
 
@@ -382,6 +396,13 @@ class ResidualStream:
             self.materialize(ctx)
         self.pending = delta
         self.pending_scale = scale
+
+    def add_pair(self, first, second, ctx: StepContext, scale: float = 1.0) -> None:
+        """The stream gains scale * (first + second): two branches that read the same rows. Either may be None, when
+        its producer has added it through a ResidualSink."""
+        self.add(first if first is not None else second, ctx, scale)
+        if first is not None and second is not None:
+            self.pending2 = second
 
     def sink_for(self, norm: Norm | None, ctx: StepContext, scale: float = 1.0) -> "ResidualSink | None":
         """A sink for the part that runs next, when `norm` (the norm that will read the stream
@@ -402,6 +423,13 @@ class ResidualStream:
             return ready[1]
         if prepared is not None and prepared[0] is norm and self.pending is None:
             return prepared[1] if rows_ok else prepared[1].tensor(ctx)
+        if self.pending2 is not None:
+            if norm.takes_pair:
+                out = norm.add_norm(self.resid, self.pending, self.rows, ctx, delta_scale=self.pending_scale,
+                                    delta2=self.pending2)
+                self.pending = self.pending2 = None
+                return out
+            self.materialize(ctx)
         if self.pending is not None and self.pending_scale != 1.0:
             out = norm.add_norm(self.resid, self.pending, self.rows, ctx, delta_scale=self.pending_scale)
         else:
@@ -412,8 +440,8 @@ class ResidualStream:
     def materialize(self, ctx: StepContext) -> torch.Tensor:
         if self.pending is not None:
             from ..kernels import ops
-            ops.residual_add(self.resid, self.pending, self.rows, self.pending_scale)
-            self.pending = None
+            ops.residual_add(self.resid, self.pending, self.rows, self.pending_scale, delta2=self.pending2)
+            self.pending = self.pending2 = None
         return self.resid
 
 

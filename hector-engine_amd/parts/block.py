@@ -8,6 +8,9 @@ the rows of the norm that follows (parts.base.ResidualSink).
 residual_scale m (1 unless given): x = x + m * mixer(norm1(x)); x = x + m * feed_forward(norm2(x)).
 A layer without a feed-forward (feed_forward None) is the first line alone.
 
+The "parallel_residual" block has one norm, whose rows both branches read:
+    x = x + (mixer(norm(x)) + feed_forward(norm(x))).
+
 The "post_norm" block norms what a branch returns and nothing it reads:
     x = x + m * norm1(mixer(x));  x = x + m * norm2(feed_forward(x))."""
 from __future__ import annotations
@@ -66,6 +69,62 @@ class PreNormBlock(Block):
         delta = self.feed_forward.forward(n, ctx)
         ctx.sink = None
         stream.add(delta, ctx, m)
+
+
+@register_part("block", "parallel_residual")
+class ParallelResidualBlock(Block):
+    """A layer whose mixer and feed-forward read the same rows, n = norm(x), and are added together:
+        x = x + (mixer(n) + feed_forward(n)).
+    A layer without a feed-forward is x = x + mixer(n). In steps of few rows each branch's last product adds into
+    the stream itself (the second one also leaves the rows of the norm that follows); otherwise the next norm's
+    launch adds both. names: norm, mixer, feed_forward (suffixes of the parts' prefixes)."""
+
+    def __init__(self, params: dict, prefix: str, env: BuildEnv):
+        super().__init__(prefix, env)
+        names = param(params, "names", dict)
+        self.norm = build_part("norm", param(params, "norm", PartSpec), prefix + names["norm"] + ".", env)
+        self.mixer = build_part("mixer", param(params, "mixer", PartSpec), prefix + names["mixer"] + ".", env)
+        self.feed_forward = None
+        if param(params, "feed_forward", PartSpec, None) is not None:
+            self.feed_forward = build_part("feed_forward", param(params, "feed_forward", PartSpec),
+                                           prefix + names["feed_forward"] + ".", env)
+
+    def children(self):
+        return [p for p in (self.norm, self.mixer, self.feed_forward) if p is not None]
+
+    def first_norm(self):
+        return self.norm
+
+    def tensor_specs(self):
+        specs = {}
+        for c in self.children():
+            specs.update(c.tensor_specs())
+        return specs
+
+    def bind(self, tensors):
+        for c in self.children():
+            c.bind(tensors)
+
+    def forward(self, stream: ResidualStream, ctx: StepContext, cache: LayerCache) -> None:
+        after, ff = ctx.next_norm, self.feed_forward
+        rows_ok = self.mixer.accepts_normed_rows and (ff is None or ff.accepts_normed_rows)
+        n = stream.normed(self.norm, ctx, rows_ok)
+        # the rows this sink leaves are of a stream that still lacks the feed-forward: nobody reads them
+        # (where nothing follows, this block's own norm stands in for the one they would be made for)
+        ctx.sink = stream.sink_for(after if ff is None else after or self.norm, ctx)
+        first = self.mixer.forward(n, ctx, cache)
+        ctx.sink = None
+        if ff is None:
+            stream.add(first, ctx)
+            return
+        stream.prepared = stream.ready = None
+        if first is not None:
+            second = ff.forward(n, ctx)
+        else:
+            ctx.sink = stream.sink_for(after, ctx)
+            second = ff.forward(n, ctx)
+            ctx.sink = None
+        stream.add_pair(first, second, ctx)
 
 
 @register_part("block", "sandwich_norm")

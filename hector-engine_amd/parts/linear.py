@@ -273,7 +273,7 @@ class Linear:
                 ops.splitk_reduce_residual(sink.stream.resid, partial, bias, gain, xg, sq, rows, splits,
                                            out_pieces=out_pieces, scale=sink.scale,
                                            dyt_bias=dyt[0] if dyt else None, dyt_alpha=dyt[1] if dyt else None)
-        sink.stream.prepared = (sink.norm, NormedRows(xg, sq, eps, rows, out_pieces))
+        sink.stream.prepared = (sink.norm, NormedRows(xg, sq, eps, rows, out_pieces, bool(dyt)))
         return None
 
     def gated_silu_rows(self, rows: int, ctx: StepContext, act: torch.dtype) -> bool:
@@ -285,9 +285,9 @@ class Linear:
         """out[rows, N/2] = silu(gate) * up in one kernel, for a weight whose rows alternate gate
         and up (gate i at row 2i, its up at 2i + 1), where gated_silu_rows() says so. x: a tensor,
         NormedRows or PieceRows; out_pieces: out is shaped and written piece-major. act: the
-        constants of another gated activation ({alpha, limit, up_shift} as ops.silu_mul takes them)."""
+        constants of another gated activation ({alpha, limit, up_shift, cubic} as ops.silu_mul takes them)."""
         act = act or {}
-        consts = (act.get("alpha", 1.0), act.get("limit", 0.0), act.get("up_shift", 0.0))
+        consts = (act.get("alpha", 1.0), act.get("limit", 0.0), act.get("up_shift", 0.0), act.get("cubic", 0.0))
         act, a, scale, pieces = _operand(x)
         if not self.gated_silu_rows(rows, ctx, act):
             raise ValueError("Linear.gated_silu: not for these rows (ask gated_silu_rows)")

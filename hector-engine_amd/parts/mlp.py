@@ -6,9 +6,13 @@ src/graph_builder.cpp:1400-1414).
 
 activation "clamped_swiglu" is the same feed-forward through a bounded gate:
 g' = min(g, limit), u' = clamp(u, -limit, limit), act = g' * sigmoid(alpha * g') * (u' + 1), with
-the parameters `limit` and `alpha` (1.702 unless given). names: the suffixes of its tensors
+the parameters `limit` and `alpha` (1.702 unless given). activation "gelu_tanh" has gelu's tanh form for the
+gate, 0.5 g (1 + tanh(c (g + a g^3))) with c = sqrt(2 / pi) and a = 0.044715, which is
+g * sigmoid(2 c g + 2 c a g^3). names: the suffixes of its tensors
 (gate, up, down)."""
 from __future__ import annotations
+
+import math
 
 import torch
 
@@ -37,6 +41,9 @@ class GatedMLP(FeedForward):
             if limit <= 0:
                 raise ValueError(f"gated_mlp: limit {limit} must be positive")
             self.act = {"alpha": param(params, "alpha", float, 1.702), "limit": limit, "up_shift": 1.0}
+        elif act == "gelu_tanh":
+            two_c = 2.0 * math.sqrt(2.0 / math.pi)
+            self.act = {"alpha": two_c, "cubic": 0.044715 * two_c}
         else:
             raise ValueError(f"gated_mlp: unsupported activation '{act}'")
         names = param(params, "names", dict, {})

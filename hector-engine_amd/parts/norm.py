@@ -44,13 +44,17 @@ class DynamicTanh(Norm):
     stands where a norm would and computes neither a mean nor a variance, so no row is reduced and no
     pair of products has a row scale to carry; where a product adds into the stream itself (steps of
     up to 64 rows), its epilogue computes this norm in full. Computed in fp32 on the fp32 residual stream, fused with the
-    pending (scaled) residual add. names: suffixes of its tensors (weight, bias, alpha)."""
+    pending (scaled) residual add of one branch output or two. scale (1 unless given) multiplies the result: it is
+    folded into weight and bias, which are then kept in 32-bit. names: suffixes of its tensors (weight, bias, alpha)."""
+
+    takes_pair = True
 
     def __init__(self, params: dict, prefix: str, env: BuildEnv):
         super().__init__(prefix, env)
         self.size = param(params, "size", int)
         names = param(params, "names", dict, {})
         self._names = {k: tensor_name(prefix, names, k, k) for k in ("weight", "bias", "alpha")}
+        self.scale = param(params, "scale", float, 1.0)
         self.weight = self.bias = self.alpha = None
 
     def tensor_specs(self):
@@ -64,13 +68,16 @@ class DynamicTanh(Norm):
         self.weight, self.bias, self.alpha = tensors[n["weight"]], tensors[n["bias"]], tensors[n["alpha"]]
         if not (self.weight.dtype == self.bias.dtype == self.alpha.dtype):
             raise TypeError(f"{self.prefix}: weight, bias and alpha are stored in different dtypes")
+        if self.scale != 1.0:
+            self.weight, self.bias = self.weight.float() * self.scale, self.bias.float() * self.scale
+            self.alpha = self.alpha.float()
 
     def carried(self):
         return self.weight, 1.0, self.bias, self.alpha
 
-    def add_norm(self, resid, delta, rows, ctx: StepContext, want_out: bool = True, delta_scale: float = 1.0):
+    def add_norm(self, resid, delta, rows, ctx: StepContext, want_out: bool = True, delta_scale: float = 1.0, delta2=None):
         out = ctx.alloc((rows, self.size)) if want_out else None
-        ops.add_dyt(resid, delta, self.weight, self.bias, self.alpha, out, rows, delta_scale)
+        ops.add_dyt(resid, delta, self.weight, self.bias, self.alpha, out, rows, delta_scale, delta2)
         return out
 
 

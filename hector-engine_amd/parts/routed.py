@@ -1,6 +1,6 @@
 """A routed feed-forward (mixture of experts): each token uses `top` of its experts.
 
-    z = W_router n                    fp32, E + I outputs: E experts with weights, then I without
+    z = W_router n (+ bias)           fp32, E + I outputs: E experts with weights, then I without
     s = softmax(z)                    over all outputs
     c = s + correction                the choice is made on c, the weights on s
     the outputs are cut into `groups` equal runs of neighbours, each run ranked by the largest c it
@@ -22,16 +22,19 @@ half of the experts reads only the chosen experts' rows of the same matrices (op
 Options: `normalize` divides the chosen outputs' weights by their sum (the softmax over the chosen logits
 alone; the choice itself is the same, the softmax being monotone); `shared` = {"feed_forward": PartSpec, "name":
 suffix of its prefix, "gate": suffix of a stored vector of hidden_size or None} adds an expert that every token
-uses, out += sigmoid(gate . n) * shared(n) (gate None: out += shared(n)), the dot product in fp32.
-names: the suffixes of its tensors (router, correction; expert e's are 'e<e>.' + gate / up / down).
+uses, out += sigmoid(gate . n) * shared(n) (gate None: out += shared(n)), the dot product in fp32; `router_bias` adds a
+stored number an output to the logits. A shared expert without a gate whose activation is the experts' own joins their
+fused matrices as columns of weight 1: it costs no launch of its own.
+names: the suffixes of its tensors (router, router_bias, correction; expert e's are 'e<e>.' + gate / up / down).
 """
 from __future__ import annotations
 
 import torch
 
 from ..kernels import ops
-from .base import BuildEnv, FeedForward, PartSpec, StepContext, TensorSpec, build_part, param, register_part, tensor_name
+from .base import BuildEnv, FeedForward, NormedRows, PartSpec, StepContext, TensorSpec, build_part, param, register_part, tensor_name
 from .linear import Linear
+from .mlp import GatedMLP
 
 # rows whose gate and up columns are held at once in a long prompt step
 _ROW_CHUNK = 4096
@@ -51,6 +54,8 @@ class RoutedExperts(FeedForward):
         self.keep = param(params, "keep_groups", int, self.groups)
         self.has_correction = param(params, "correction", bool, True)
         self.normalize = param(params, "normalize", bool, False)
+        self.has_bias = param(params, "router_bias", bool, False)
+        self.bias = None
         shared = param(params, "shared", dict, None)
         self.shared = self.shared_gate = self._shared_gate = None
         if shared:
@@ -60,6 +65,14 @@ class RoutedExperts(FeedForward):
         self.limit = param(params, "limit", float, 0.0)
         self.alpha = param(params, "alpha", float, 1.702 if self.limit > 0 else 1.0)
         self.up_shift = param(params, "up_shift", float, 1.0 if self.limit > 0 else 0.0)
+        # columns of a shared expert that run as part of the experts' own products
+        act = {"alpha": self.alpha, "limit": self.limit, "up_shift": self.up_shift, "cubic": 0.0}
+        self.shared_cols = 0
+        if isinstance(self.shared, GatedMLP) and not self._shared_gate \
+                and {**{"alpha": 1.0, "limit": 0.0, "up_shift": 0.0, "cubic": 0.0}, **self.shared.act} == act:
+            self.shared_cols = self.shared.inter
+        # rows prepared for a norm may come as they are, where they owe nothing
+        self.accepts_normed_rows = self.shared is None or self.shared_cols > 0
         E = self.real + self.identity
         if self.real <= 0 or self.identity < 0 or self.inter <= 0:
             raise ValueError("routed_experts: experts and intermediate_size must be positive, identity_experts not negative")
@@ -72,6 +85,7 @@ class RoutedExperts(FeedForward):
         names = param(params, "names", dict, {})
         self._router = tensor_name(prefix, names, "router", "router.weight")
         self._correction = tensor_name(prefix, names, "correction", "router.correction")
+        self._bias = tensor_name(prefix, names, "router_bias", "router.bias")
         self._expert = names.get("expert", "experts.{e}.")
         self._sub = {k: names.get(k, d) for k, d in (("gate", "gate_proj.weight"), ("up", "up_proj.weight"),
                                                      ("down", "down_proj.weight"))}
@@ -87,6 +101,8 @@ class RoutedExperts(FeedForward):
         specs = {self._router: TensorSpec((self.real + self.identity, self.hidden))}
         if self.has_correction:
             specs[self._correction] = TensorSpec((self.real + self.identity,))
+        if self.has_bias:
+            specs[self._bias] = TensorSpec((self.real + self.identity,), ("normal", 0.1))
         for e in range(self.real):
             specs[self._name(e, "gate")] = TensorSpec((self.inter, self.hidden))
             specs[self._name(e, "up")] = TensorSpec((self.inter, self.hidden))
@@ -104,18 +120,23 @@ class RoutedExperts(FeedForward):
         # the router's sums are 32-bit whatever the run's precision: its matrix is kept in float32
         self.router = tensors[self._router].to(torch.float32).contiguous()
         self.correction = tensors[self._correction] if self.has_correction else None
+        self.bias = tensors[self._bias] if self.has_bias else None
         gu, downs = [], []
         for e in range(self.real):
             g, u = tensors.pop(self._name(e, "gate")), tensors.pop(self._name(e, "up"))
             # gate i of an expert at row 2i of its stretch, its up at 2i + 1
             gu.append(torch.stack([g, u], 1).reshape(2 * self.inter, self.hidden))
             downs.append(tensors.pop(self._name(e, "down")))
+        if self.shared_cols:
+            g, u, dn = (tensors.pop(self.shared._names[k]) for k in ("gate", "up", "down"))
+            gu.append(torch.stack([g, u], 1).reshape(2 * self.shared_cols, self.hidden))
+            downs.append(dn)
         if self.identity:
             # the identity experts' share rides through the down product on an identity block
             downs.append(torch.eye(self.hidden, dtype=downs[0].dtype, device=downs[0].device))
         self.gate_up = Linear(torch.cat(gu, 0).contiguous())
         self.down = Linear(torch.cat(downs, 1).contiguous())
-        if self.shared is not None:
+        if self.shared is not None and not self.shared_cols:
             self.shared.bind(tensors)
         if self._shared_gate:
             self.shared_gate = tensors[self._shared_gate].reshape(-1).contiguous()
@@ -124,11 +145,11 @@ class RoutedExperts(FeedForward):
         """Whether the step runs through the chosen experts alone (kernels.ops.chosen_experts): bfloat16 with the
         fast kernels, sizes in multiples of 8, and so few rows that they cannot choose more than half of the
         experts. (The 32-bit path keeps the products over all experts, whose sums do not depend on the batch.)"""
-        return (ctx.env.fast_kernels and x.dtype == torch.bfloat16 and self.gate_up.weight.dtype == torch.bfloat16
-                and self.inter % 8 == 0 and self.hidden % 8 == 0 and 2 * rows * self.top <= self.real)
+        return (ctx.env.fast_kernels and ctx.env.dtype == torch.bfloat16 and self.gate_up.weight.dtype == torch.bfloat16
+                and self.inter % 8 == 0 and self.shared_cols % 8 == 0 and self.hidden % 8 == 0 and 2 * rows * self.top <= self.real)
 
     def forward(self, x, ctx: StepContext):
-        if self.shared is None:
+        if self.shared is None or self.shared_cols:
             return self._routed(x, ctx, True)
         rows = ctx.rows
         routed = self._routed(x, ctx, False)
@@ -141,25 +162,33 @@ class RoutedExperts(FeedForward):
         return out
 
     def _routed(self, x, ctx: StepContext, may_sink: bool):
-        rows, real, I = ctx.rows, self.real, self.inter
+        rows, real, I, S = ctx.rows, self.real, self.inter, self.shared_cols
+        # rows a product has left for this norm: read as they lie where they owe nothing (and no identity expert wants
+        # them row by row), else made into a tensor
+        pieces = isinstance(x, NormedRows) and x.finished and x.pieces and not self.identity
+        given = x                                    # what the experts' first product reads
+        if isinstance(x, NormedRows):
+            x = x.scaled if pieces else x.tensor(ctx)
+            given = given if pieces else x
         dense = ctx.alloc((rows, real + 1), torch.float32)
         ids = ctx.alloc((rows, self.top), torch.int32)
         weights = ctx.alloc((rows, self.top), torch.float32)
         # the router's product (fp32 sums over the rows as they are) and the choice, one launch
         ops.route_tokens(dense, ids, weights, None, self.correction, rows, real, self.groups, self.keep,
-                         self.top, self.scale, x=x, router=self.router, normalize=self.normalize)
-        cols = real * I + (self.hidden if self.identity else 0)
+                         self.top, self.scale, x=x, router=self.router, normalize=self.normalize, bias=self.bias, x_pieces=pieces)
+        cols = real * I + S + (self.hidden if self.identity else 0)
         act = {"alpha": self.alpha, "limit": self.limit, "up_shift": self.up_shift}
         if self._few_rows(rows, x, ctx):
             # the rows of the step choose at most half of the experts: only those experts' weights are read
-            h = ctx.alloc((rows * self.top, I))
+            h = ctx.alloc((rows * (self.top * I + S),))
             out = ctx.alloc((rows, self.hidden))
-            ops.chosen_experts(out, h, x, self.gate_up.weight, self.down.weight, ids, weights, dense, rows, real, I, **act)
+            ops.chosen_experts(out, h, x, self.gate_up.weight, self.down.weight, ids, weights, dense, rows, real, I,
+                               shared=S, x_pieces=pieces, **act)
             return out
         if rows <= _ROW_CHUNK:
-            gu = self.gate_up(x, rows, ctx)
+            gu = self.gate_up(given, rows, ctx)
             h = ctx.alloc((rows, cols))
-            ops.routed_act(h, gu, dense, x if self.identity else None, rows, real, I, **act)
+            ops.routed_act(h, gu, dense, x if self.identity else None, rows, real, I, shared=S, **act)
             return self.down(h, rows, ctx, sink=ctx.take_sink() if may_sink else None)
         out = ctx.alloc((rows, self.hidden))
         for r0 in range(0, rows, _ROW_CHUNK):
@@ -167,7 +196,8 @@ class RoutedExperts(FeedForward):
             turn = ctx.scratch.mark()
             gu = self.gate_up(x[r0:r0 + n], n, ctx)
             h = ctx.alloc((n, cols))
-            ops.routed_act(h, gu, dense[r0:r0 + n], x[r0:r0 + n] if self.identity else None, n, real, I, **act)
+            ops.routed_act(h, gu, dense[r0:r0 + n], x[r0:r0 + n] if self.identity else None, n, real, I, shared=S,
+                           **act)
             self.down(h, n, ctx, out=out[r0:r0 + n])
             ctx.scratch.release(turn)
         return out

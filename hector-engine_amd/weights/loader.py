@@ -31,7 +31,7 @@ def check_against(expected: dict[str, TensorSpec], found: dict[str, tuple],
     missing = sorted(n for n in expected if n not in found)
     unexpected = sorted(n for n in found if n not in expected and n not in allowed_extra)
     wrong = sorted((n, tuple(expected[n].shape), tuple(found[n])) for n in expected
-                   if n in found and tuple(found[n]) != tuple(expected[n].shape))
+                   if n in found and not expected[n].matches(tuple(found[n])))
     if not (missing or unexpected or wrong):
         return
     lines = ["the model folder's tensors do not match the configuration:"]

@@ -126,7 +126,7 @@ def init_moments(name: str, init: tuple) -> tuple[float, float]:
 def random_tensor(name: str, spec: TensorSpec, seed: int, dtype: torch.dtype, device) -> torch.Tensor:
     device = torch.device(device)
     key = tensor_key(seed, name)
-    shape = tuple(spec.shape)
+    shape = spec.random_shape()
     n = int(np.prod(shape, dtype=np.int64)) if shape else 1
     on_gpu = device.type == "cuda"
     if on_gpu:
