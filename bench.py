@@ -4,7 +4,7 @@ token ids) on one MI355X, with prefill and roofline figures on the same line.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L] [--shape 7b|32b|72b]
                     [--context C] [--prompt P]
-    python bench.py --design volonex | penasun | butolorn | domorax      (another measurement: see below)
+    python bench.py --design volonex | penasun | butolorn | domorax | dofipel      (another measurement: see below)
 
 The default is the 7B shape; --shape runs the same measurement at the layer sizes of
 Qwen2.5-32B (context 8192, prompts of 512 to 2048 tokens, batches 1 / 8 / 64) or
@@ -29,7 +29,7 @@ leaves its first run and its thermal-low samples out: OPTIMIZATION_NOTES.md:114-
 every timed run, the earlier ones still show it.
 
 --design volonex (or penasun; butolorn and domorax are measured beside Penasun, the other design whose layers carry
-a state of fixed size) leaves the run above aside and measures that design beside Qwen2 at equal layer
+a state of fixed size, and dofipel beside Domorax, the other design with attention through latents) leaves the run above aside and measures that design beside Qwen2 at equal layer
 sizes (random weights, bf16, four layers of each of a few sizes that resemble real models' layers): prompt
 tokens a second for one prompt of 2,048 tokens, decoded tokens a second at batch 8 and batch 1 behind such
 prompts, and, from a second pass with an event pair around every launch, the mean time of each kind of
@@ -184,6 +184,28 @@ def domorax_configs(sz):
     return penasun, config_from_dict(domorax)
 
 
+def dofipel_configs(sz):
+    """(Domorax configuration, Dofipel configuration) of one set of layer sizes. Domorax is the design beside it: both
+    have attention through latents and a routed feed-forward with a shared expert. The Dofipel layers are an attention
+    through latents (Domorax's: 64 rotated dims, a latent of 192, but every earlier position and a gate on its output) with a
+    dense feed-forward of the Qwen2 layer's width, a second one that reads the first one's latents, an attention over a
+    window of 1,024 with capped scores and a distance table, and a latent attention of its own; the last three route 4 of
+    16 experts, each a quarter of the Qwen2 feed-forward wide, beside a shared expert of that width."""
+    from hector_engine_amd.registry import config_from_dict
+    _, domorax = domorax_configs(sz)
+    latent = dict(heads=sz["heads"], dim=sz["dim"], rot_dim=64, vdim=sz["vdim"], kv_rank=192, scale=(sz["dim"] + 64) ** -0.5,
+                  rot=dict(base=10000.0, dims=64))
+    attention = dict(heads=sz["heads"], kv_heads=sz["kv_heads"], dim=sz["dim"], vdim=sz["vdim"], scale=sz["dim"] ** -0.5,
+                     softcap=30.0, bias_max=256, mask=dict(size=1024))
+    dense = dict(kind="dense", ff=sz["ff"])
+    moe = dict(kind="moe", expert=dict(ff=sz["ff"] // 4), router=dict(experts=16, top=4), shared=dict(ff=sz["ff"] // 4))
+    layers = [dict(type="latent_attention", mixer=latent, mlp=dense),
+              dict(type="latent_attention", mixer=dict(latent, kv_from=0), mlp=moe),
+              dict(type="attention", mixer=attention, mlp=moe), dict(type="latent_attention", mixer=latent, mlp=moe)]
+    dofipel = dict(architecture="Dofipel", vocab=DESIGN_VOCAB, width=sz["width"], logit_scale=1.5, norm=dict(eps=1e-6), layers=layers)
+    return domorax, config_from_dict(dofipel)
+
+
 def compare_designs(args) -> int:
     import torch
     import hector_engine_amd as he
@@ -262,13 +284,13 @@ def compare_designs(args) -> int:
         return out
 
     result = {}
-    beside = "penasun" if args.design in ("butolorn", "domorax") else "qwen2"
+    beside = {"butolorn": "penasun", "domorax": "penasun", "dofipel": "domorax"}.get(args.design, "qwen2")
     chosen = [n for n in DESIGN_SIZES if not args.design_sizes or n in args.design_sizes.split(",")]
     for name in chosen:
         sz = DESIGN_SIZES[name]
         result[name] = {"sizes": sz}
         configs = {"volonex": design_configs, "penasun": penasun_configs, "butolorn": butolorn_configs,
-                   "domorax": domorax_configs}[args.design](sz)
+                   "domorax": domorax_configs, "dofipel": dofipel_configs}[args.design](sz)
         for design, config in zip((beside, args.design), configs):
             progress(f"{name} {design}")
             result[name][design] = measure(config, False)
@@ -309,9 +331,9 @@ def main() -> int:
     ap.add_argument("--no-tune", action="store_true",
                     help="leave the library's default kernels for the tall matrix products")
     ap.add_argument("--design-sizes", default="", help=f"with --design: only these of {', '.join(DESIGN_SIZES)}")
-    ap.add_argument("--design", choices=["volonex", "penasun", "butolorn", "domorax"], default=None,
-                    help="instead of the run above: this design beside Qwen2 (butolorn, domorax: beside Penasun) at equal layer sizes, prompt and "
-                         "one-token steps, throughput and mean time per kind of kernel")
+    ap.add_argument("--design", choices=["volonex", "penasun", "butolorn", "domorax", "dofipel"], default=None,
+                    help="instead of the run above: this design beside Qwen2 (butolorn, domorax: beside Penasun; dofipel: beside "
+                         "Domorax) at equal layer sizes, prompt and one-token steps, throughput and mean time per kind of kernel")
     args = ap.parse_args()
     if args.design:
         return compare_designs(args)

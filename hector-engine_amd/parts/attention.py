@@ -473,11 +473,13 @@ class Attention(Mixer):
         rows, H, KVH, hd = ctx.rows, self.Hk, self.KVHk, self.pd
         q, gate = self._encoded_q(x, ctx, cache)
         out = ctx.alloc((rows, H * hd))
-        floats = ops.attention_decode_workspace_floats(rows, H, KVH, hd, ctx.max_keys)
+        # the most keys a query sees: no slices of the keys are launched (or given room) beyond them
+        most = min([ctx.max_keys] + [reach + ops.PAGE_TOKENS for reach in (self.window, self.chunk) if reach > 0])
+        floats = ops.attention_decode_workspace_floats(rows, H, KVH, hd, most)
         ws = ctx.alloc((max(floats, 1),), torch.float32)
         ops.attention_decode(out, q, cache.kpool, cache.vpool, ctx.positions, ctx.row_seq,
                              ctx.seq_slot, cache.page_table, rows, H, KVH, hd, self.window,
-                             self.scale, ctx.max_keys, ws, chunk=self.chunk, sinks=self.sinks,
+                             self.scale, most, ws, chunk=self.chunk, sinks=self.sinks,
                              gate=gate if self.head_gate else None, slopes=self.slopes, cap=self.score_cap,
                              table=self.table)
         return self._project(out, rows, ctx, gate)
