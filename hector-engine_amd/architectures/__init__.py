@@ -1,2 +1,2 @@
 """Architectures known to the registry."""
-from . import butolorn, dofipel, domorax, penasun, qwen2, volonex  # noqa: F401
+from . import bobevik, butolorn, dofipel, domorax, penasun, qwen2, volonex  # noqa: F401

@@ -5,10 +5,13 @@
 #include "hector_kernels.h"
 
 // out[t, :] = table[ids[t], :] * scale as fp32 (scale 1: the row as it is); an id outside
-// [0, V) gives a zero row (reference: kernels/linear.cu:36-69).
+// [0, V) gives a zero row (reference: kernels/linear.cu:36-69). norm_w: the row is then divided by
+// sqrt(mean(x^2) + eps) and multiplied by norm_w (each thread goes over the elements it has written).
 template <typename T>
 __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ table,
-                                 const int32_t* __restrict__ ids, int D, int V, float scale) {
+                                 const int32_t* __restrict__ ids, int D, int V, float scale,
+                                 const void* __restrict__ norm_w, int w_dtype, float eps) {
+  __shared__ float scratch[16];
   const int64_t t = blockIdx.x;
   const int id = ids[t];
   float* o = out + t * (int64_t)D;
@@ -17,6 +20,7 @@ __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ 
     return;
   }
   const T* row = table + (int64_t)id * D;
+  float ss = 0.f;      // of the elements this thread has written
   if (sizeof(T) == 2 && (D & 7) == 0 && (((uintptr_t)table | (uintptr_t)out) & 15) == 0) {
     // eight elements a thread and turn: one 16-byte load, two 16-byte stores
     for (int i = 8 * threadIdx.x; i < D; i += 8 * blockDim.x) {
@@ -30,24 +34,39 @@ __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ 
       }
       *reinterpret_cast<float4*>(o + i) = make_float4(f[0], f[1], f[2], f[3]);
       *reinterpret_cast<float4*>(o + i + 4) = make_float4(f[4], f[5], f[6], f[7]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = fmaf(f[j], f[j], ss);
     }
+    if (norm_w == nullptr) return;
+    const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)D + eps);
+    for (int i = 8 * threadIdx.x; i < D; i += 8 * blockDim.x)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[i + j] = o[i + j] * inv * load_param(norm_w, i + j, w_dtype);
     return;
   }
-  for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = to_float(row[i]) * scale;
+  for (int i = threadIdx.x; i < D; i += blockDim.x) {
+    const float f = to_float(row[i]) * scale;
+    o[i] = f;
+    ss = fmaf(f, f, ss);
+  }
+  if (norm_w == nullptr) return;
+  const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)D + eps);
+  for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = o[i] * inv * load_param(norm_w, i, w_dtype);
 }
 
 extern "C" int he_embedding(void* out_f32, const void* table, const void* ids, int rows, int D,
-                            int V, int table_dtype, float scale, void* stream) {
+                            int V, int table_dtype, float scale, const void* norm_w, int w_dtype, float eps,
+                            void* stream) {
   HE_REQUIRE(rows >= 0 && D > 0 && V > 0, "he_embedding: bad sizes rows=%d D=%d V=%d", rows, D, V);
   if (rows == 0) return 0;
   const int threads = D >= 1024 ? 256 : (D >= 256 ? 128 : 64);
   hipStream_t s = (hipStream_t)stream;
   if (table_dtype == HE_BF16)
     embedding_kernel<bf16_t><<<rows, threads, 0, s>>>((float*)out_f32, (const bf16_t*)table,
-                                                      (const int32_t*)ids, D, V, scale);
+                                                      (const int32_t*)ids, D, V, scale, norm_w, w_dtype, eps);
   else if (table_dtype == HE_F32)
     embedding_kernel<float><<<rows, threads, 0, s>>>((float*)out_f32, (const float*)table,
-                                                     (const int32_t*)ids, D, V, scale);
+                                                     (const int32_t*)ids, D, V, scale, norm_w, w_dtype, eps);
   else
     HE_REQUIRE(false, "he_embedding: unknown dtype %d", table_dtype);
   return he_check_launch("he_embedding");

@@ -6,7 +6,7 @@
 #pragma once
 #include <stdint.h>
 
-#define HE_ABI_VERSION 30
+#define HE_ABI_VERSION 31
 
 #ifdef __cplusplus
 extern "C" {
@@ -26,9 +26,10 @@ int he_fill_random_integers(void* out_i32, int64_t n, uint64_t key, int64_t high
 int he_cast(void* out, const void* in, int64_t n, int in_dtype, int out_dtype, void* stream);
 
 // ---- row-wise ------------------------------------------------------------
-// out[t, :] = table[ids[t], :] * scale in fp32.
+// out[t, :] = table[ids[t], :] * scale in fp32; with norm_w [D] the row is then divided by
+// sqrt(mean(x^2) + eps) and multiplied by it.
 int he_embedding(void* out_f32, const void* table, const void* ids, int rows, int D, int V,
-                 int table_dtype, float scale, void* stream);
+                 int table_dtype, float scale, const void* norm_w, int w_dtype, float eps, void* stream);
 int he_gather_rows_f32(void* out, const void* src, const void* rows, int n_out, int D, int n_src,
                        void* stream);
 // resid += scale * (delta + delta2) (delta2 may be null).
@@ -137,7 +138,10 @@ int he_qkv_rope_cache(void* q_out, void* kpool, void* vpool, const void* q_in, c
                       const void* row_seq, const void* seq_slot, const void* page_table,
                       int max_blocks, int num_pages, const void* inv_freq, int rotary_dim, int rows,
                       int H, int KVH, int hd, int hd_in, int vd_in, int interleaved, float mscale,
-                      float q_coef, int q_every, int dtype, void* stream);
+                      float q_coef, int q_every, int unit, float unit_eps, const void* v_first,
+                      int64_t v_stride, float v_lambda, int dtype, void* stream);
+// unit: every head of q and k is divided by sqrt(mean(x^2) + unit_eps) as well (bias and rotation as before). v_first
+// (rows of KVH * vd_in values, v_stride elements apart, or null): v <- (1 - v_lambda) v + v_lambda v_first.
 // hd: head size of q_out and of the cache pages. hd_in, vd_in (0: hd): head sizes of the q/k rows and
 // of the v rows that come in (at most hd; q_out is padded with zeros, the pages keep their zeros).
 // interleaved: frequency i turns the pair (2i, 2i + 1), not (i, i + rotary_dim / 2). mscale multiplies
@@ -319,6 +323,12 @@ int he_sample_rows(void* out_i32, const void* logits_f32, int rows, int V, int64
 int he_add_normed(void* resid_f32, const void* delta, int delta_dtype, const void* post_weight, float post_eps,
                   const void* next_weight, float next_eps, int w_dtype, void* out, int out_dtype, int rows, int D,
                   void* stream);
+// The same of two branches side by side, delta = scale * (rmsnorm(a) * w_a + rmsnorm(b) * w_b) with pair_eps (gains of
+// pair_dtype); without resid_f32, out = delta.
+int he_add_normed_pair(void* resid_f32, const void* a, const void* b, int delta_dtype, const void* w_a, const void* w_b,
+                       int pair_dtype, float pair_eps, float scale, const void* post_weight, float post_eps,
+                       const void* next_weight, float next_eps, int w_dtype, void* out, int out_dtype, int rows, int D,
+                       void* stream);
 // kind: 0 relu^2, 1 gelu (tanh form), 2 silu, 3 relu
 int he_unary_act(void* out, const void* x, int64_t n, int kind, int dtype, void* stream);
 // out[r, j] = act(x[r, j]) * table[ids[r], offset + j], j < W
@@ -343,6 +353,21 @@ int he_delta_scan(void* y_f32, const void* q, const void* k, const void* v, int6
                   int64_t state_offset, const void* cu_seqlens, const void* seq_slot, int rows, int num_seqs, int H, int G,
                   int d, int e, float q_scale, float unit_eps, void* workspace_f32, int64_t workspace_floats, int dtype,
                   void* stream);
+
+// ---- a memory per head that fades by a constant factor a token (decay_memory.hip) -------------------
+// y_f32 [rows, H dv] from q, k [rows, H dk] and v [rows, H dv] (views of rows in_stride elements apart):
+// S <- decay_h S + k v^T, y = S^T q. act: q, k and v pass SiLU first; then the first 2 * half dims of every head of q
+// and k turn by positions[row] * inv_freq[i] (pair (i, i + half)), and k is multiplied by k_scale. powers_f32
+// [H][65]: decay_h^0 .. decay_h^64. S (fp32, he_decay_state_floats floats) lives at byte state_offset of the
+// sequence's row of the state area, zeros at a sequence's start, and is carried on. max_q_len: the most rows of a
+// sequence in this step. workspace_f32: he_decay_workspace_floats floats on a 16-byte boundary. dk up to 512.
+int64_t he_decay_state_floats(int H, int dk, int dv);
+int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv, int half);
+int he_decay_scan(void* y_f32, const void* q, const void* k, const void* v, int64_t in_stride, const void* powers_f32,
+                  int act, float k_scale, const void* inv_freq_f32, int half, const void* positions, void* state,
+                  int64_t state_stride, int64_t state_offset, const void* cu_seqlens, const void* seq_slot, int rows,
+                  int num_seqs, int max_q_len, int H, int dk, int dv, void* workspace_f32, int64_t workspace_floats,
+                  int dtype, void* stream);
 
 // ---- norms over parts of a row (group_norm.hip) --------------------------------------------------------
 // resid += delta_scale * gn(delta) with gn the RMS norm in `groups` equal consecutive parts times weight (delta null:

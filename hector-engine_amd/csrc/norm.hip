@@ -543,6 +543,123 @@ __global__ void add_normed_vec_kernel(float* __restrict__ resid, const TD* __res
   }
 }
 
+// Two branches side by side, each normed over the row with a gain of its own:
+//   x = scale * (a / rms(a) * w_a + b / rms(b) * w_b),   rms(z) = sqrt(mean(z^2) + pair_eps).
+// With resid given, x then goes the way of a branch output above (normed by post_w if given, added to resid, and out
+// = what the next reader wants of it); without, out = x. Everything in fp32 registers between the loads and out. VEC:
+// runs of four neighbouring elements a thread (what add_normed_vec_kernel asks of widths and addresses).
+template <typename TD, typename TO, bool VEC>
+__global__ void add_normed_pair_kernel(float* __restrict__ resid, const TD* __restrict__ a, const TD* __restrict__ b,
+                                       const void* __restrict__ w_a, const void* __restrict__ w_b, int pair_dtype,
+                                       float pair_eps, float scale, const void* __restrict__ post_w, float post_eps,
+                                       const void* __restrict__ next_w, float next_eps, int w_dtype,
+                                       TO* __restrict__ out, int D) {
+  __shared__ float scratch[16], scratch_b[16];
+  constexpr int RUN = VEC ? 4 : 1;
+  const int64_t row = blockIdx.x;
+  auto at = [&](int e) { return VEC ? (threadIdx.x + (e / 4) * blockDim.x) * 4 + e % 4 : threadIdx.x + e * blockDim.x; };
+  auto load = [&](float* x, const auto* p) {
+#pragma unroll
+    for (int e = 0; e < PN_EPT; e += RUN) {
+      const int i = at(e);
+      if constexpr (VEC) {
+        if (i < D) pn_load4(x + e, p + i);
+        else x[e] = x[e + 1] = x[e + 2] = x[e + 3] = 0.f;
+      } else {
+        x[e] = i < D ? to_float(p[i]) : 0.f;
+      }
+    }
+  };
+  auto store = [&](auto* p, const float* x) {
+#pragma unroll
+    for (int e = 0; e < PN_EPT; e += RUN) {
+      const int i = at(e);
+      if (i < D) {
+        if constexpr (VEC) pn_store4(p + i, x + e);
+        else p[i] = from_float<std::remove_reference_t<decltype(*p)>>(x[e]);
+      }
+    }
+  };
+  float x[PN_EPT], z[PN_EPT];
+  load(x, a + row * D);
+  load(z, b + row * D);
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int e = 0; e < PN_EPT; ++e) {
+    sa = fmaf(x[e], x[e], sa);
+    sb = fmaf(z[e], z[e], sb);
+  }
+  const float ia = scale / sqrtf(block_sum(sa, scratch) / (float)D + pair_eps);
+  const float ib = scale / sqrtf(block_sum(sb, scratch_b) / (float)D + pair_eps);
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < PN_EPT; ++e) {
+    const int i = at(e);
+    if (i < D) x[e] = x[e] * ia * load_param(w_a, i, pair_dtype) + z[e] * ib * load_param(w_b, i, pair_dtype);
+    ss = fmaf(x[e], x[e], ss);
+  }
+  if (resid == nullptr) {
+    store(out + row * D, x);
+    return;
+  }
+  const float inv = post_w ? 1.0f / sqrtf(block_sum(ss, scratch) / (float)D + post_eps) : 1.f;
+  load(z, resid + row * D);
+  ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < PN_EPT; ++e) {
+    const int i = at(e);
+    if (i < D) x[e] = z[e] + x[e] * inv * (post_w ? load_param(post_w, i, w_dtype) : 1.f);
+    ss = fmaf(x[e], x[e], ss);
+  }
+  store(resid + row * D, x);
+  if (out == nullptr) return;
+  if (next_w) {
+    const float inv2 = 1.0f / sqrtf(block_sum(ss, scratch_b) / (float)D + next_eps);
+#pragma unroll
+    for (int e = 0; e < PN_EPT; ++e) {
+      const int i = at(e);
+      if (i < D) x[e] = x[e] * inv2 * load_param(next_w, i, w_dtype);
+    }
+  }
+  store(out + row * D, x);
+}
+
+extern "C" int he_add_normed_pair(void* resid_f32, const void* a, const void* b, int delta_dtype, const void* w_a,
+                                  const void* w_b, int pair_dtype, float pair_eps, float scale, const void* post_weight,
+                                  float post_eps, const void* next_weight, float next_eps, int w_dtype, void* out,
+                                  int out_dtype, int rows, int D, void* stream) {
+  HE_REQUIRE(rows >= 0 && D > 0, "he_add_normed_pair: bad sizes rows=%d D=%d", rows, D);
+  HE_REQUIRE(D <= PN_EPT * 1024, "he_add_normed_pair: width %d above %d", D, PN_EPT * 1024);
+  HE_REQUIRE(a && b && w_a && w_b && (resid_f32 || out), "he_add_normed_pair: a branch, a gain or the result is missing");
+  HE_REQUIRE((w_dtype == HE_F32 || w_dtype == HE_BF16) && (pair_dtype == HE_F32 || pair_dtype == HE_BF16),
+             "he_add_normed_pair: bad weight dtype");
+  HE_REQUIRE((delta_dtype == HE_F32 || delta_dtype == HE_BF16) && (out_dtype == HE_F32 || out_dtype == HE_BF16),
+             "he_add_normed_pair: unknown dtype");
+  if (rows == 0) return 0;
+  int threads = 64;
+  while (threads < 1024 && PN_EPT * threads < D) threads <<= 1;
+  while (threads < 256 && 4 * threads < D) threads <<= 1;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = D % 4 == 0 && (((uintptr_t)resid_f32 | (uintptr_t)a | (uintptr_t)b | (uintptr_t)out) & 15) == 0;
+#define PN_PAIR(TD, TO, VEC)                                                                                            \
+  add_normed_pair_kernel<TD, TO, VEC><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)a, (const TD*)b, w_a, w_b, \
+                                                               pair_dtype, pair_eps, scale, post_weight, post_eps,      \
+                                                               next_weight, next_eps, w_dtype, (TO*)out, D)
+#define PN_PAIR_VEC(TD, TO)          \
+  do {                               \
+    if (vec) PN_PAIR(TD, TO, true);  \
+    else PN_PAIR(TD, TO, false);     \
+  } while (0)
+  const bool db = delta_dtype == HE_BF16, ob = out_dtype == HE_BF16;
+  if (db && ob) PN_PAIR_VEC(bf16_t, bf16_t);
+  else if (db) PN_PAIR_VEC(bf16_t, float);
+  else if (ob) PN_PAIR_VEC(float, bf16_t);
+  else PN_PAIR_VEC(float, float);
+#undef PN_PAIR_VEC
+#undef PN_PAIR
+  return he_check_launch("he_add_normed_pair");
+}
+
 extern "C" int he_add_normed(void* resid_f32, const void* delta, int delta_dtype, const void* post_weight, float post_eps,
                              const void* next_weight, float next_eps, int w_dtype, void* out, int out_dtype, int rows,
                              int D, void* stream) {

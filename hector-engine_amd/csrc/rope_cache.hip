@@ -8,6 +8,10 @@
 //   y[i]       = x[i] * cos a - x[i + r/2] * sin a
 //   y[i + r/2] = x[i] * sin a + x[i + r/2] * cos a
 // and dims >= r pass through. All of it in fp32.
+//
+// Two options of the same pass: every head of q and of k divided by its own root mean square (no gain; a rotation does
+// not change it, so it is formed from the rows as they come), and values mixed with an earlier layer's values of the
+// same row, v <- (1 - lambda) v + lambda v_first.
 #include "cache_layout.h"
 #include "hector_kernels.h"
 
@@ -18,6 +22,16 @@
 __device__ __forceinline__ float he_query_temperature(int pos, float coef, int every) {
   return every > 0 ? fmaf(coef, logf((float)((pos + 1) / every + 1)), 1.f) : 1.f;
 }
+
+// unit: heads of q and k are divided by sqrt(mean(x^2) + eps). v_first: rows of another layer's values as they were
+// projected (KVH * vd_in of them, no bias, `stride` elements apart) that join the own ones with the factor lambda.
+struct RopeExtras {
+  int unit;
+  float eps;
+  const void* v_first;
+  int64_t v_stride;
+  float v_lambda;
+};
 
 // hd: the head size of q_out and of the cache pages; hd_in <= hd, vd_in <= hd: the head sizes of the
 // projected q/k and v rows (a mixer whose keys and values differ in width keeps both in pages of
@@ -33,8 +47,9 @@ __global__ void qkv_rope_cache_kernel(
     const int32_t* __restrict__ row_seq, const int32_t* __restrict__ seq_slot,
     const int32_t* __restrict__ page_table, int max_blocks, int num_pages,
     const float* __restrict__ inv_freq, int rotary_dim, int H, int KVH, int hd, int hd_in, int vd_in,
-    int interleaved, float mscale, float q_coef, int q_every) {
+    int interleaved, float mscale, float q_coef, int q_every, RopeExtras ex) {
   __shared__ float cs[2][ROPE_MAX_HALF];
+  extern __shared__ float inv_rms[];     // ex.unit: one number a head of q, then of k
   const int64_t row = blockIdx.x;
   const int seq = row_seq[row];
   if (seq < 0) return;  // padding row
@@ -47,6 +62,23 @@ __global__ void qkv_rope_cache_kernel(
     sincos_angle(a, &sn, &c);
     cs[0][i] = c * mscale;
     cs[1][i] = sn * mscale;
+  }
+  if (ex.unit) {
+    const int lane = threadIdx.x & 63, heads = H + (k_in ? KVH : 0);
+    for (int h = threadIdx.x >> 6; h < heads; h += blockDim.x >> 6) {
+      const bool of_q = h < H;
+      const int base = (of_q ? h : h - H) * hd_in;
+      const TI* in = (of_q ? q_in : k_in) + row * in_stride + base;
+      const void* bias = of_q ? q_bias : k_bias;
+      float ss = 0.f;
+      for (int d = lane; d < hd_in; d += 64) {
+        float x = to_float(in[d]);
+        if (bias) x += load_param(bias, base + d, bias_dtype);
+        ss = fmaf(x, x, ss);
+      }
+      ss = wave_sum(ss);
+      if (lane == 0) inv_rms[h] = 1.f / sqrtf(ss / (float)hd_in + ex.eps);
+    }
   }
   __syncthreads();
   // the two dims of pair j
@@ -62,6 +94,7 @@ __global__ void qkv_rope_cache_kernel(
       const int h = it / per_head;
       const int j = it - h * per_head;
       const int base = h * hd_in, obase = h * hd;
+      const float mul = ex.unit ? q_mul * inv_rms[h] : q_mul;
       if (j < half) {
         const int d0 = pair_mul * j, d1 = d0 + pair_step;
         float x0 = to_float((in + base + d0)[0]);
@@ -71,8 +104,8 @@ __global__ void qkv_rope_cache_kernel(
           x1 += load_param(q_bias, base + d1, bias_dtype);
         }
         const float c = cs[0][j], sn = cs[1][j];
-        out[obase + d0] = from_float<T>((x0 * c - x1 * sn) * q_mul);
-        out[obase + d1] = from_float<T>((x0 * sn + x1 * c) * q_mul);
+        out[obase + d0] = from_float<T>((x0 * c - x1 * sn) * mul);
+        out[obase + d1] = from_float<T>((x0 * sn + x1 * c) * mul);
       } else {
         const int d = rotary_dim + (j - half);
         float x = 0.f;
@@ -80,7 +113,7 @@ __global__ void qkv_rope_cache_kernel(
           x = to_float((in + base + d)[0]);
           if (q_bias) x += load_param(q_bias, base + d, bias_dtype);
         }
-        out[obase + d] = from_float<T>(x * q_mul);
+        out[obase + d] = from_float<T>(x * mul);
       }
     }
   }
@@ -100,6 +133,7 @@ __global__ void qkv_rope_cache_kernel(
       const int base = h * hd_in;
       T* out = kpool + ((int64_t)page * KVH + h) * he_k_page_elems(hd);   // the page, in operand order
       const int KS = he_k_steps(hd);
+      const float mul = ex.unit ? inv_rms[H + h] : 1.f;
       if (j < half) {
         const int d0 = pair_mul * j, d1 = d0 + pair_step;
         float x0 = to_float((in + base + d0)[0]);
@@ -109,13 +143,13 @@ __global__ void qkv_rope_cache_kernel(
           x1 += load_param(k_bias, base + d1, bias_dtype);
         }
         const float c = cs[0][j], sn = cs[1][j];
-        out[he_k_index(off, d0, KS)] = from_float<T>(x0 * c - x1 * sn);
-        out[he_k_index(off, d1, KS)] = from_float<T>(x0 * sn + x1 * c);
+        out[he_k_index(off, d0, KS)] = from_float<T>((x0 * c - x1 * sn) * mul);
+        out[he_k_index(off, d1, KS)] = from_float<T>((x0 * sn + x1 * c) * mul);
       } else {
         const int d = rotary_dim + (j - half);
         float x = to_float((in + base + d)[0]);
         if (k_bias) x += load_param(k_bias, base + d, bias_dtype);
-        out[he_k_index(off, d, KS)] = from_float<T>(x);
+        out[he_k_index(off, d, KS)] = from_float<T>(x * mul);
       }
     }
   }
@@ -127,6 +161,8 @@ __global__ void qkv_rope_cache_kernel(
       const int d = it - h * vd_in;
       float x = to_float((in + it)[0]);
       if (v_bias) x += load_param(v_bias, it, bias_dtype);
+      if (ex.v_first)
+        x = (1.f - ex.v_lambda) * x + ex.v_lambda * to_float(((const TI*)ex.v_first)[row * ex.v_stride + it]);
       vpool[((int64_t)page * KVH + h) * he_v_page_elems(hd) + he_v_index(off, d, he_v_tiles(hd))] =
           from_float<T>(x);
     }
@@ -165,8 +201,10 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
     const int32_t* __restrict__ positions, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ seq_slot, const int32_t* __restrict__ page_table, int max_blocks,
     int num_pages, const float* __restrict__ inv_freq, int rotary_dim, int rows, int H, int KVH,
-    int hd, int hd_in, int vd_in, int interleaved, float mscale, int v_span, float q_coef, int q_every) {
+    int hd, int hd_in, int vd_in, int interleaved, float mscale, int v_span, float q_coef, int q_every,
+    RopeExtras ex) {
   __shared__ float cs[2][ROPE_MAX_HALF];
+  extern __shared__ float squares[];     // ex.unit: an item's share of its head's sum of squares
   const int v_blocks = (int)gridDim.x - rows;   // they come first: theirs is the longest chain of dependent loads
   if ((int)blockIdx.x < v_blocks) {
     // ---- v: the runs of tokens that begin in rows [r0, r0 + v_span). In a step of few rows (one token a
@@ -193,9 +231,20 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
         // row and is dropped): they go out together
 #pragma unroll
         for (int i = 0; i < 8; ++i) vals[i] = v_in[(int64_t)(r + min(i, n - 1)) * in_stride + e];
+        if (ex.v_first) {
+          uint16_t firsts[8];
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            firsts[i] = ((const uint16_t*)ex.v_first)[(int64_t)(r + min(i, n - 1)) * ex.v_stride + e];
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            vals[i] = float_to_bf16_bits((1.f - ex.v_lambda) * (bf16_bits_to_float(vals[i]) + b) +
+                                         ex.v_lambda * bf16_bits_to_float(firsts[i]));
+          }
+        }
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-          if (v_bias) vals[i] = float_to_bf16_bits(bf16_bits_to_float(vals[i]) + b);
+          if (v_bias && !ex.v_first) vals[i] = float_to_bf16_bits(bf16_bits_to_float(vals[i]) + b);
           if (i >= n) vals[i] = 0;
         }
         uint16_t* out = vpool + ((int64_t)page * KVH + h) * he_v_page_elems(hd) + he_v_index(off, d, NT);
@@ -278,12 +327,44 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
     cs[0][i] = c * mscale;
     cs[1][i] = sn * mscale;
   }
+  if (ex.unit) {
+    auto square = [&](int it, const Item& im, const uint4 (&raw)[4]) {
+      float ss = 0.f;
+#pragma unroll
+      for (int half_of = 0; half_of < 2; ++half_of) {       // the item's own elements, then its partners'
+        if (half_of == 1 && (!im.rotated || interleaved)) break;
+        float x[8], b[8];
+        unpack8(raw[half_of], x);
+        unpack8(raw[2 + half_of], b);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss = fmaf(x[i] + b[i], x[i] + b[i], ss);
+      }
+      squares[it] = ss;
+    };
+    if (has_first) square(threadIdx.x, first, first_raw);
+    for (int it = threadIdx.x + blockDim.x; it < items; it += blockDim.x) {
+      const Item im = item(it);
+      uint4 raw[4];
+      load(im, raw);
+      square(it, im, raw);
+    }
+  }
   __syncthreads();
+  // what a head is multiplied by: the shares of its items, added in their order
+  auto unit_mul = [&](const Item& im) {
+    if (!ex.unit) return 1.f;
+    const int per_head = im.is_q ? per_head_q : per_head_k;
+    const float* p = squares + (im.is_q ? 0 : q_items) + im.h * per_head;
+    float ss = 0.f;
+    for (int i = 0; i < per_head; ++i) ss += p[i];
+    return 1.f / sqrtf(ss / (float)hd_in + ex.eps);
+  };
   const bool cache_ok = page >= 0 && page < num_pages;
   const int off = pos & (HE_PAGE_TOKENS - 1);
   const int KS = he_k_steps(hd);
   const float q_mul = he_query_temperature(pos, q_coef, q_every);
   const bool tempered = q_mul != 1.f;
+  const bool scaled = tempered || ex.unit;
   auto finish = [&](const Item& im, const uint4 (&raw)[4]) {
     // where the eight elements from dim d on go: the q row, or the cache page in operand order
     uint16_t* out;
@@ -294,6 +375,7 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
       out = kpool + ((int64_t)page * KVH + im.h) * he_k_page_elems(hd);
     }
     auto at = [&](int d) { return out + (im.is_q ? d : he_k_index(off, d, KS)); };
+    const float mul = (im.is_q ? q_mul : 1.f) * unit_mul(im);
     float x0[8], x1[8], b0[8], b1[8];
     unpack8(raw[0], x0);
     unpack8(raw[2], b0);
@@ -306,9 +388,9 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
         y[2 * i] = a0 * c - a1 * sn;
         y[2 * i + 1] = a0 * sn + a1 * c;
       }
-      if (im.is_q && tempered) {
+      if (scaled) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) y[i] *= q_mul;
+        for (int i = 0; i < 8; ++i) y[i] *= mul;
       }
       *reinterpret_cast<uint4*>(at(im.j)) = pack8(y);
     } else if (im.rotated) {
@@ -322,18 +404,17 @@ __global__ __launch_bounds__(1024) void qkv_rope_cache_vec_kernel(
         y0[i] = a0 * c - a1 * sn;
         y1[i] = a0 * sn + a1 * c;
       }
-      if (im.is_q && tempered) {
+      if (scaled) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-          y0[i] *= q_mul;
-          y1[i] *= q_mul;
+          y0[i] *= mul;
+          y1[i] *= mul;
         }
       }
       *reinterpret_cast<uint4*>(at(im.j)) = pack8(y0);
       *reinterpret_cast<uint4*>(at(im.j + half)) = pack8(y1);
     } else {
-      if (im.bias || (im.is_q && tempered)) {
-        const float mul = im.is_q ? q_mul : 1.f;
+      if (im.bias || scaled) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) x0[i] = (x0[i] + b0[i]) * mul;
         *reinterpret_cast<uint4*>(at(im.j)) = pack8(x0);
@@ -358,7 +439,9 @@ extern "C" int he_qkv_rope_cache(void* q_out, void* kpool, void* vpool, const vo
                                  const void* seq_slot, const void* page_table, int max_blocks,
                                  int num_pages, const void* inv_freq, int rotary_dim, int rows,
                                  int H, int KVH, int hd, int hd_in, int vd_in, int interleaved,
-                                 float mscale, float q_coef, int q_every, int dtype, void* stream) {
+                                 float mscale, float q_coef, int q_every, int unit, float unit_eps,
+                                 const void* v_first, int64_t v_stride, float v_lambda, int dtype,
+                                 void* stream) {
   HE_REQUIRE(rows >= 0 && H > 0 && KVH >= 0 && hd > 0, "he_qkv_rope_cache: bad sizes");
   if (hd_in <= 0) hd_in = hd;
   if (vd_in <= 0) vd_in = hd;
@@ -374,16 +457,26 @@ extern "C" int he_qkv_rope_cache(void* q_out, void* kpool, void* vpool, const vo
   HE_REQUIRE(k_in == nullptr || (kpool && vpool && page_table && max_blocks > 0 && KVH > 0),
              "he_qkv_rope_cache: cache arguments missing");
   HE_REQUIRE(dtype == HE_BF16 || dtype == HE_F32, "he_qkv_rope_cache: unknown dtype %d", dtype);
+  HE_REQUIRE(v_first == nullptr || (k_in != nullptr && v_stride >= (int64_t)KVH * vd_in),
+             "he_qkv_rope_cache: rows of other values are %lld wide, not %d", (long long)v_stride, KVH * vd_in);
+  HE_REQUIRE(H + KVH <= 8192, "he_qkv_rope_cache: %d heads", H + KVH);
   if (rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const int threads = 256;
+  RopeExtras ex;
+  ex.unit = unit;
+  ex.eps = unit_eps;
+  ex.v_first = v_first;
+  ex.v_stride = v_stride;
+  ex.v_lambda = v_lambda;
+  const size_t head_floats = unit ? sizeof(float) * (H + KVH) : 0;
 #define ROPE_LAUNCH(T, TI)                                                                      \
-  qkv_rope_cache_kernel<T, TI><<<rows, threads, 0, s>>>(                                        \
+  qkv_rope_cache_kernel<T, TI><<<rows, threads, head_floats, s>>>(                                      \
       (T*)q_out, (T*)kpool, (T*)vpool, (const TI*)q_in, (const TI*)k_in, (const TI*)v_in,       \
       in_stride, q_bias, k_bias, v_bias, bias_dtype,                                            \
       (const int32_t*)positions, (const int32_t*)row_seq, (const int32_t*)seq_slot,             \
       (const int32_t*)page_table, max_blocks, num_pages, (const float*)inv_freq, rotary_dim, H, \
-      KVH, hd, hd_in, vd_in, interleaved, mscale, q_coef, q_every)
+      KVH, hd, hd_in, vd_in, interleaved, mscale, q_coef, q_every, ex)
   const bool vec_ok = dtype == HE_BF16 &&
                       (q_bias == nullptr || bias_dtype == HE_BF16) &&
                       ((interleaved ? rotary_dim : rotary_dim >> 1) & 7) == 0 && ((hd - rotary_dim) & 7) == 0 &&
@@ -394,16 +487,17 @@ extern "C" int he_qkv_rope_cache(void* q_out, void* kpool, void* vpool, const vo
   if (vec_ok) {
     const int rot8 = (interleaved ? rotary_dim : rotary_dim >> 1) >> 3;
     const int items = H * (rot8 + ((hd - rotary_dim) >> 3)) + (k_in ? KVH * (rot8 + ((hd_in - rotary_dim) >> 3)) : 0);
+    HE_REQUIRE(!unit || items <= 12288, "he_qkv_rope_cache: %d heads are too many to norm", H + KVH);
     const int vec_threads = min(1024, max(64, (items + 63) / 64 * 64));
     const int v_span = rows <= 128 ? 1 : 8;
     const int v_blocks = k_in ? (rows + v_span - 1) / v_span : 0;
-    qkv_rope_cache_vec_kernel<<<rows + v_blocks, vec_threads, 0, s>>>(
+    qkv_rope_cache_vec_kernel<<<rows + v_blocks, vec_threads, unit ? sizeof(float) * items : 0, s>>>(
         (uint16_t*)q_out, (uint16_t*)kpool, (uint16_t*)vpool, (const uint16_t*)q_in,
         (const uint16_t*)k_in, (const uint16_t*)v_in, in_stride, (const uint16_t*)q_bias,
         (const uint16_t*)k_bias, (const uint16_t*)v_bias, (const int32_t*)positions,
         (const int32_t*)row_seq, (const int32_t*)seq_slot, (const int32_t*)page_table, max_blocks,
         num_pages, (const float*)inv_freq, rotary_dim, rows, H, KVH, hd, hd_in, vd_in, interleaved, mscale, v_span, q_coef,
-        q_every);
+        q_every, ex);
   } else if (dtype == HE_BF16) {
     ROPE_LAUNCH(bf16_t, bf16_t);
   } else {

@@ -76,6 +76,13 @@ class DecoderModel:
         self.mix_coeffs = [tensors[name] for name in self.depth_mix or []]
         for p in self.parts():
             p.bind(tensors)
+        # parts that keep rows for the whole step
+        self.keepers, todo = [], list(self.parts())
+        while todo:
+            p = todo.pop(0)
+            if p.step_columns():
+                self.keepers.append((p, p.step_columns()))
+            todo += p.children()
 
     # -- cache ----------------------------------------------------------------
     def run_plans(self) -> list[RunPlan]:
@@ -95,6 +102,8 @@ class DecoderModel:
         ctx.tokens = ids
         resid = self.embedding.forward(ids, rows, ctx)
         stream = ResidualStream(resid, rows)
+        ctx.room = {p: ctx.alloc((rows, columns)) for p, columns in self.keepers}
+        ctx.handed = {}
         embedded = None
         if any(entry.add_embedding for entry in self.schedule):
             # the embedding's output, kept for the runs that start again from it

@@ -16,7 +16,7 @@ _lib = None
 
 _CSRC = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "csrc")
 
-EXPECTED_ABI = 30
+EXPECTED_ABI = 31
 
 c_int, c_i64, c_f32, c_ptr = ctypes.c_int, ctypes.c_int64, ctypes.c_float, ctypes.c_void_p
 
@@ -26,7 +26,7 @@ _SIGNATURES = {
     "he_fill_random": [c_ptr, c_i64, c_int, ctypes.c_uint64, c_ptr, c_f32, c_f32, c_ptr],
     "he_fill_random_integers": [c_ptr, c_i64, ctypes.c_uint64, c_i64, c_ptr],
     "he_cast": [c_ptr, c_ptr, c_i64, c_int, c_int, c_ptr],
-    "he_embedding": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_f32, c_ptr],
+    "he_embedding": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_f32, c_ptr, c_int, c_f32, c_ptr],
     "he_gather_rows_f32": [c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_ptr],
     "he_residual_add": [c_ptr, c_ptr, c_ptr, c_i64, c_int, c_f32, c_ptr],
     "he_silu_mul": [c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_ptr],
@@ -55,7 +55,8 @@ _SIGNATURES = {
                                   c_int, c_int, c_f32, c_ptr, c_ptr, c_ptr],
     "he_qkv_rope_cache": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_ptr,
                           c_int, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_ptr, c_int, c_int,
-                          c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_int, c_int, c_ptr],
+                          c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_int, c_int, c_f32, c_ptr, c_i64, c_f32, c_int,
+                          c_ptr],
     "he_conv_state": [c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_int, c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_ptr, c_ptr,
                       c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr],
     "he_ssm_state_floats": [c_int, c_int, c_int],
@@ -69,12 +70,18 @@ _SIGNATURES = {
     "he_mlstm_scan": [c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_i64, c_i64, c_ptr, c_ptr, c_int, c_int,
                       c_int, c_int, c_int, c_f32, c_int, c_int, c_ptr, c_int, c_f32, c_ptr],
     "he_add_normed": [c_ptr, c_ptr, c_int, c_ptr, c_f32, c_ptr, c_f32, c_int, c_ptr, c_int, c_int, c_int, c_ptr],
+    "he_add_normed_pair": [c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_ptr, c_int, c_f32, c_f32, c_ptr, c_f32, c_ptr, c_f32, c_int,
+                           c_ptr, c_int, c_int, c_int, c_ptr],
     "he_unary_act": [c_ptr, c_ptr, c_i64, c_int, c_int, c_ptr],
     "he_token_gate": [c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr],
     "he_sigmoid_gate": [c_ptr, c_ptr, c_i64, c_int, c_int, c_int, c_int, c_f32, c_int, c_ptr],
     "he_scaled_sum": [c_ptr, c_ptr, c_ptr, c_i64, c_f32, c_f32, c_int, c_ptr],
     "he_route_tokens": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_int, c_ptr, c_int, c_int, c_int, c_int,
                         c_int, c_int, c_int, c_f32, c_int, c_ptr, c_int, c_int, c_ptr],
+    "he_decay_state_floats": [c_int, c_int, c_int],
+    "he_decay_workspace_floats": [c_int, c_int, c_int, c_int, c_int, c_int, c_int],
+    "he_decay_scan": [c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_int, c_f32, c_ptr, c_int, c_ptr, c_ptr, c_i64, c_i64, c_ptr,
+                      c_ptr, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr, c_i64, c_int, c_ptr],
     "he_delta_state_floats": [c_int, c_int, c_int],
     "he_delta_scan": [c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_i64, c_i64, c_ptr, c_ptr,
                       c_int, c_int, c_int, c_int, c_int, c_int, c_f32, c_f32, c_ptr, c_i64, c_int, c_ptr],
@@ -127,6 +134,8 @@ _RESTYPES = {
     "he_attention_plain_workspace_floats": c_i64,
     "he_ssm_state_floats": c_i64,
     "he_mlstm_state_floats": c_i64,
+    "he_decay_state_floats": c_i64,
+    "he_decay_workspace_floats": c_i64,
     "he_delta_state_floats": c_i64,
     "he_delta_workspace_floats": c_i64,
     "he_gemm_plain_workspace_floats": c_i64,

@@ -74,17 +74,20 @@ def cast(out, src) -> None:
 
 
 @_op("embedding")
-def embedding(out_f32, table, ids, rows: int, scale: float = 1.0) -> None:
-    """out[t] = table[ids[t]] * scale in fp32."""
+def embedding(out_f32, table, ids, rows: int, scale: float = 1.0, norm_weight=None, norm_eps: float = 0.0) -> None:
+    """out[t] = table[ids[t]] * scale in fp32; with norm_weight [D] it is then RMS-normed with that gain."""
     V, D = table.shape
     _need(table, "table")
     _need(out_f32, "out", torch.float32)
     _need(ids, "ids", torch.int32)
     if out_f32.numel() < rows * D or ids.numel() < rows:
         raise ValueError("embedding: buffers smaller than the row count")
+    if norm_weight is not None:
+        _need(norm_weight, "norm_weight", shape=(D,))
     L = _lib.load()
     _lib.check(L.he_embedding(out_f32.data_ptr(), table.data_ptr(), ids.data_ptr(), rows, D, V,
-                              dtype_code(table.dtype), float(scale), _stream()))
+                              dtype_code(table.dtype), float(scale), _ptr(norm_weight),
+                              dtype_code(norm_weight.dtype) if norm_weight is not None else F32, float(norm_eps), _stream()))
 
 
 @_op("gather_rows")
@@ -515,13 +518,15 @@ def splitk_reduce(out, partial, bias, M: int, splits: int) -> None:
 def qkv_rope_cache(q_out, kpool, vpool, qkv, q_cols: int, kv_cols: int, bias, positions, row_seq,
                    seq_slot, page_table, inv_freq, rotary_dim: int, rows: int, H: int, KVH: int,
                    hd: int, write_kv: bool, *, key_dim: int = 0, value_dim: int = 0,
-                   interleaved: bool = False, mscale: float = 1.0, q_temp=None) -> None:
+                   interleaved: bool = False, mscale: float = 1.0, q_temp=None, unit_eps=None, v_mix=None) -> None:
     """qkv: [rows, q_cols + kv_cols + v_cols (+ more)] projected rows without bias; bias (optional)
     covers those columns. Rotated q goes to q_out [rows, H*hd]; k, v go into the pools at
     (slot, position) when write_kv. hd is the head size of q_out and of the cache pages; key_dim and
     value_dim (0: hd) are the head sizes of the q/k and of the v columns, at most hd (q_out is then
     padded with zeros, the pages keep the zeros they were made with). interleaved: frequency i turns
-    the dims (2i, 2i + 1) instead of (i, i + rotary_dim / 2); mscale multiplies cos and sin."""
+    the dims (2i, 2i + 1) instead of (i, i + rotary_dim / 2); mscale multiplies cos and sin. unit_eps (a
+    number): every head of q and k is divided by sqrt(mean(x^2) + unit_eps). v_mix = (lambda, first): the values become
+    (1 - lambda) v + lambda first, first a view [rows, KVH * value_dim] of wider rows."""
     _need(qkv, "qkv")
     _need(q_out, "q_out")
     if qkv.dtype != q_out.dtype:
@@ -568,6 +573,12 @@ def qkv_rope_cache(q_out, kpool, vpool, qkv, q_cols: int, kv_cols: int, bias, po
             vb = qb + (q_cols + kv_cols) * bes
     if rotary_dim:
         _need(inv_freq, "inv_freq", torch.float32, (rotary_dim // 2,))
+    first = None
+    if v_mix is not None:
+        first = v_mix[1]
+        if not write_kv or not first.is_cuda or first.dtype != qkv.dtype or first.dim() != 2 or first.shape[0] < rows \
+                or first.shape[1] != v_cols or first.stride(1) != 1:
+            raise ValueError(f"qkv_rope_cache: v_mix takes a [rows, {v_cols}] view in the rows' dtype, where values are written")
     L = _lib.load()
     _lib.check(L.he_qkv_rope_cache(
         q_out.data_ptr(), _ptr(kpool) if write_kv else None, _ptr(vpool) if write_kv else None,
@@ -575,7 +586,9 @@ def qkv_rope_cache(q_out, kpool, vpool, qkv, q_cols: int, kv_cols: int, bias, po
         seq_slot.data_ptr(), _ptr(page_table) if write_kv else None, max_blocks, num_pages,
         _ptr(inv_freq) if rotary_dim else None, rotary_dim, rows, H, KVH if write_kv else 0, hd,
         kd, vd, int(interleaved), float(mscale), float(q_temp[0]) if q_temp else 0.0,
-        int(q_temp[1]) if q_temp else 0, dtype_code(q_out.dtype), _stream()))
+        int(q_temp[1]) if q_temp else 0, int(unit_eps is not None), float(unit_eps or 0.0), _ptr(first),
+        first.stride(0) if first is not None else 0, float(v_mix[0]) if v_mix is not None else 0.0,
+        dtype_code(q_out.dtype), _stream()))
 
 
 @_op("conv_state")
@@ -663,6 +676,62 @@ def gated_group_norm(out, y, z, weight, rows: int, parts: int, eps: float, gate_
     _lib.check(L.he_gated_group_norm(out.data_ptr(), y.data_ptr(), z.data_ptr(), z.stride(0), weight.data_ptr(),
                                      dtype_code(weight.dtype), rows, W, parts, float(eps), 2 if gate_after == "silu" else int(bool(gate_after)),
                                      float(out_scale), dtype_code(out.dtype), _stream()))
+
+
+DECAY_POWERS = 65        # powers of a decay that decay_scan reads: 0 .. 64
+
+
+def decay_state_floats(H: int, dk: int, dv: int) -> int:
+    """Floats of a sequence's fading memories (the value dims padded to fours)."""
+    return int(_lib.load().he_decay_state_floats(H, dk, dv))
+
+
+def decay_workspace_floats(rows: int, num_seqs: int, max_q_len: int, H: int, dk: int, dv: int, half: int) -> int:
+    """Floats of workspace decay_scan wants for a step of these sizes (0: none)."""
+    return int(_lib.load().he_decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv, half))
+
+
+@_op("decay_scan")
+def decay_scan(y, q, k, v, powers, state, state_offset: int, positions, cu_seqlens, seq_slot, rows: int, num_seqs: int,
+               max_q_len: int, H: int, dk: int, dv: int, *, act: bool = False, k_scale: float = 1.0, inv_freq=None,
+               workspace=None) -> None:
+    """y (fp32 [rows, H dv]) = the memories that fade by a constant factor a token, S <- decay S + k v^T, y = S^T q, over
+    q, k [rows, H dk] and v [rows, H dv] (views of rows of one buffer, unit stride along the columns). powers: fp32
+    [H, 65], decay^0 .. decay^64. act: q, k and v pass SiLU first; inv_freq (fp32 [r/2] or None): the first r dims of
+    every head of q and k are rotated at the row's position; k is multiplied by k_scale. The state [H][dk][dv'] lives at
+    byte state_offset of a sequence's row of `state` and is carried on. max_q_len: the most rows of a sequence.
+    workspace: fp32, decay_workspace_floats elements or more (None: made here)."""
+    _need(y, "y", torch.float32, (None, H * dv))
+    stride = q.stride(0)
+    for name, t, width in (("q", q, H * dk), ("k", k, H * dk), ("v", v, H * dv)):
+        if not t.is_cuda or t.dtype != q.dtype or t.dim() != 2 or t.shape[1] != width or t.stride(1) != 1 \
+                or t.stride(0) != stride or t.shape[0] < rows:
+            raise ValueError(f"decay_scan: {name} must be a [rows, {width}] view of rows {stride} elements apart")
+    if y.shape[0] < rows:
+        raise ValueError("decay_scan: y has fewer rows than the step")
+    _need(powers, "powers", torch.float32, (H, DECAY_POWERS))
+    if state.dtype != torch.uint8 or state.dim() != 2 or state.stride(1) != 1 \
+            or state.shape[1] < state_offset + 4 * decay_state_floats(H, dk, dv):
+        raise ValueError("decay_scan: state must be uint8 [slots, bytes] with room for the memories")
+    half = 0
+    if inv_freq is not None:
+        _need(inv_freq, "inv_freq", torch.float32)
+        half = inv_freq.numel()
+    for name, t, n in (("positions", positions, rows), ("seq_slot", seq_slot, num_seqs), ("cu_seqlens", cu_seqlens, num_seqs + 1)):
+        _need(t, name, torch.int32)
+        if t.numel() < n:
+            raise ValueError(f"decay_scan: {name} shorter than the step")
+    need = decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv, half)
+    if workspace is None and need:
+        workspace = torch.empty(need, dtype=torch.float32, device=y.device)
+    if workspace is not None:
+        _need(workspace, "workspace", torch.float32)
+    L = _lib.load()
+    _lib.check(L.he_decay_scan(y.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), stride, powers.data_ptr(), int(act),
+                               float(k_scale), _ptr(inv_freq), half, positions.data_ptr(), state.data_ptr(),
+                               state.stride(0), state_offset, cu_seqlens.data_ptr(), seq_slot.data_ptr(), rows, num_seqs,
+                               int(max_q_len), H, dk, dv, _ptr(workspace),
+                               workspace.numel() if workspace is not None else 0, dtype_code(q.dtype), _stream()))
 
 
 ACT_KINDS = {"relu2": 0, "gelu_tanh": 1, "silu": 2, "relu": 3}
@@ -871,6 +940,38 @@ def latent_cache(q_out, kpool, vpool, q, down, gain, eps: float, positions, row_
         dtype_code(gain.dtype) if down is not None else F32, float(eps), positions.data_ptr(), row_seq.data_ptr(),
         seq_slot.data_ptr(), _ptr(page_table) if down is not None else None, max_blocks, num_pages, _ptr(inv_freq) if r else None,
         int(interleaved), float(mscale), rows, H, d, r, rank, pd, dtype_code(q_out.dtype), _stream()))
+
+
+@_op("add_normed_pair")
+def add_normed_pair(resid_f32, a, b, w_a, w_b, pair_eps: float, scale: float, post_weight, post_eps: float, next_weight,
+                    next_eps: float, out, rows: int) -> None:
+    """delta = scale * (rmsnorm(a) * w_a + rmsnorm(b) * w_b), which then joins resid as add_normed's delta does; with
+    resid None, out = delta."""
+    D = a.shape[-1]
+    if resid_f32 is not None:
+        _need(resid_f32, "resid", torch.float32)
+        if resid_f32.numel() < rows * D:
+            raise ValueError("add_normed_pair: resid smaller than the row count")
+    for name, t in (("a", a), ("b", b), ("out", out)):
+        if t is not None:
+            _need(t, name)
+            if t.shape[-1] != D or t.numel() < rows * D:
+                raise ValueError(f"add_normed_pair: {name} does not match [rows, {D}]")
+    if b.dtype != a.dtype:
+        raise TypeError("add_normed_pair: the branches must share a dtype")
+    _need(w_a, "w_a", None, (D,))
+    _need(w_b, "w_b", w_a.dtype, (D,))
+    w_dtype = None
+    for name, w in (("post_weight", post_weight), ("next_weight", next_weight)):
+        if w is not None:
+            _need(w, name, w_dtype, (D,))
+            w_dtype = w.dtype
+    L = _lib.load()
+    _lib.check(L.he_add_normed_pair(_ptr(resid_f32), a.data_ptr(), b.data_ptr(), dtype_code(a.dtype), w_a.data_ptr(),
+                                    w_b.data_ptr(), dtype_code(w_a.dtype), float(pair_eps), float(scale),
+                                    _ptr(post_weight), float(post_eps), _ptr(next_weight), float(next_eps),
+                                    dtype_code(w_dtype) if w_dtype is not None else F32, _ptr(out),
+                                    dtype_code(out.dtype) if out is not None else F32, rows, D, _stream()))
 
 
 @_op("add_normed")

@@ -29,7 +29,8 @@ Options of the same part, each off unless its parameter says otherwise:
               (eps `qk_norm_eps`) and multiplied by a stored vector of that size, k likewise; after the
               bias and before the position encoding. "head": every head of q is divided by its own root
               mean square and multiplied by one stored vector of head_dim that all heads share, every
-              head of k likewise with a second vector.
+              head of k likewise with a second vector. "unit": every head of q and of k is divided by its own root
+              mean square behind the position encoding, without a stored vector (inside the cache-write launch).
   conv_taps   K > 0: q and k pass a causal convolution per channel over the last K projected rows of the
               sequence (tensors `q_conv`, `k_conv`, [channels, K], the last column on the row's own
               input, zeros before the sequence's start, no bias), directly behind the projection and
@@ -43,6 +44,10 @@ Options of the same part, each off unless its parameter says otherwise:
               position i gains row bucket(i - j) of it. Of the B rows the first floor(B/2) =: F are the distances
               0 .. F - 1; distance n >= F has the row F + floor(ln(n / F) / ln(D / F) * (B - F)), at most B - 1
               (distance_bucket). The kernels read it spread out over the distances.
+  v_mix       {role, key}: values mixed with an earlier layer's. Role "first": this layer's values, as they are, are
+              what the other layers of the same key mix in (its own stay; the stored number is unused). Role "mix":
+              v becomes (1 - lambda) v + lambda v_first, v_first the first layer's value of the same token and lambda a
+              stored number (tensor `v_mix`); the mixed value is what the cache holds.
   q_temp      {coef, every}: the q of position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).
   score_maps  2: differential attention. A head has two queries and a kv head two keys (in the q and k
               matrices a head's rows for map 1 stand in front of its rows for map 2); the two maps are
@@ -53,7 +58,7 @@ Options of the same part, each off unless its parameter says otherwise:
               so that the heads of one (kv head, map) are neighbours, and the value rows of a kv head
               stand once for each of its maps; ops.diff_heads then joins the pairs.
   names       the suffixes of its tensors (q, k, v, o, q_bias, k_bias, v_bias, o_bias, sinks, gate,
-              lq1, lk1, lq2, lk2, q_norm, k_norm, q_conv, k_conv, distance).
+              lq1, lk1, lq2, lk2, q_norm, k_norm, q_conv, k_conv, distance, v_mix).
 """
 from __future__ import annotations
 
@@ -70,7 +75,7 @@ _NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o":
           "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
           "sinks": "sinks", "gate": "gate.weight", "lq1": "lambda_q1", "lk1": "lambda_k1", "lq2": "lambda_q2",
           "lk2": "lambda_k2", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "q_conv": "q_conv.weight", "k_conv": "k_conv.weight",
-          "distance": "distance_bias"}
+          "distance": "distance_bias", "v_mix": "v_mix"}
 from .linear import Linear
 
 
@@ -141,6 +146,9 @@ class Attention(Mixer):
         self.table_rows, self.table_far = (int(dt.get("rows", 32)), int(dt["far"])) if dt else (0, 0)
         self.table: torch.Tensor | None = None      # fp32 [H, distances]: the stored table spread out (bind)
         self.taps = None
+        vm = param(params, "v_mix", dict, None)
+        self.v_role, self.v_key = (vm["role"], str(vm["key"])) if vm else ("", "")
+        self.v_lambda = 0.0
         self.maps = param(params, "score_maps", int, 1)
         self.diff = param(params, "diff", float, 0.0)
         self.diff_eps = param(params, "diff_eps", float, 1e-6)
@@ -151,7 +159,11 @@ class Attention(Mixer):
             raise ValueError(f"attention: score_maps {self.maps} must be 1 or 2 (and 2 goes without gates and q/k norms)")
         if self.head_gate and self.out_gate:
             raise ValueError("attention: head_gate and out_gate exclude each other")
-        if self.qk_norm not in ("", "projection", "head"):
+        if self.v_role not in ("", "first", "mix"):
+            raise ValueError(f"attention: unknown v_mix role '{self.v_role}'")
+        if self.v_role and (self.maps > 1 or self.conv_taps or self.values_are_keys or not self.kv_projection):
+            raise ValueError("attention: v_mix goes without score maps, conv_taps, values 'keys' and shared caches")
+        if self.qk_norm not in ("", "projection", "head", "unit"):
             raise ValueError(f"attention: unknown qk_norm '{self.qk_norm}'")
         if param(params, "values", str, "projection") not in ("projection", "keys"):
             raise ValueError(f"attention: unknown values '{params['values']}'")
@@ -195,12 +207,17 @@ class Attention(Mixer):
         # what the fused one-token kernel and the kernels without these options do not take
         self.extras = self.chunk > 0 or self.has_sinks or self.head_gate or self.maps > 1 or self.q_temp is not None \
             or self.out_gate or self.sink_value is not None or bool(self.qk_norm) or self.conv_taps > 0 \
-            or self.values_are_keys or self.slope_span > 0 or self.score_cap > 0 or self.table_rows > 0
+            or self.values_are_keys or self.slope_span > 0 or self.score_cap > 0 or self.table_rows > 0 \
+            or bool(self.v_role)
         # rows of the gate's matrix behind q||k||v: one a head, or one for every value of every head
         self.gate_rows = self.H if self.head_gate else self.H * self.vd if self.out_gate else 0
 
     def children(self):
         return [self.position]
+
+    def step_columns(self) -> int:
+        # the projected rows, the values among them, stay until the last layer that mixes them in
+        return self.qkv.out_features if self.v_role == "first" else 0
 
     def state_bytes(self) -> int:
         # the last K - 1 projected q and k rows of the sequence, fp32
@@ -238,7 +255,9 @@ class Attention(Mixer):
             specs[n["distance"]] = TensorSpec((None, self.H), ("normal", 1.0), free=self.table_rows)
         if self.gate_rows:
             specs[n["gate"]] = TensorSpec((self.gate_rows, self.hidden))
-        if self.qk_norm:
+        if self.v_role:
+            specs[n["v_mix"]] = TensorSpec((), ("gain", 0.5, 0.1))
+        if self.qk_norm in ("projection", "head"):
             per_head = self.qk_norm == "head"
             specs[n["q_norm"]] = TensorSpec((hd if per_head else self.H * hd,), ("gain", 1.0, 0.1))
             if self.kv_projection:
@@ -296,7 +315,9 @@ class Attention(Mixer):
             self.sinks = tensors[n["sinks"]]
         elif self.sink_value is not None:
             self.sinks = torch.full((self.H,), self.sink_value, dtype=torch.float32, device=wo.device)
-        if self.qk_norm:
+        if self.v_role == "mix":
+            self.v_lambda = float(tensors[n["v_mix"]].float().item())
+        if self.qk_norm in ("projection", "head"):
             self.q_norm_w = tensors[n["q_norm"]]
             self.k_norm_w = tensors[n["k_norm"]] if self.kv_projection else None
         if self.conv_taps:
@@ -395,14 +416,26 @@ class Attention(Mixer):
         rot = self.position.rotary()
         # With a rotation (or no encoding) the bias is added inside the fused kernel;
         # any other encoding sees q and k with their bias already added.
-        fused_bias = not self.position.custom and not self.qk_norm
-        qkv = proj(x, rows, ctx, use_bias=not fused_bias)
+        # (values that other layers mix in are handed over with theirs)
+        fused_bias = not self.position.custom and self.qk_norm not in ("projection", "head") and not self.v_role
+        v_mix = None
+        if self.v_role:
+            if not writes:
+                raise RuntimeError(f"{self.prefix}: v_mix goes with a cache of its own")
+            v_at = (H + KVH) * hd
+            qkv = proj(x, rows, ctx, use_bias=not fused_bias, out=ctx.room[self] if self.v_role == "first" else None)
+            if self.v_role == "first":
+                ctx.handed[self.v_key] = qkv[:, v_at:v_at + KVH * self.vd]
+            else:
+                v_mix = (self.v_lambda, ctx.handed[self.v_key])
+        else:
+            qkv = proj(x, rows, ctx, use_bias=not fused_bias)
         if self.conv_taps or self.values_are_keys:
             qkv = self._conv_norm_rows(qkv, ctx, cache)
         elif self.qk_norm == "head":
             ops.qk_head_norm(qkv, qkv, self.q_norm_w, self.k_norm_w if writes else self.q_norm_w, H, KVH if writes else 0,
                              hd, self.qk_norm_eps, rows)
-        elif self.qk_norm:
+        elif self.qk_norm == "projection":
             # each token's q (all heads at once), and its k, by a root mean square of their own, in place
             wide = qkv.stride(0)
             if writes:
@@ -420,7 +453,8 @@ class Attention(Mixer):
                            proj.bias if fused_bias else None, ctx.positions, ctx.row_seq,
                            ctx.seq_slot, cache.page_table, inv_freq, r, rows, H, KVH, self.pd, writes,
                            key_dim=hd, value_dim=self.vd, interleaved=self.position.interleaved,
-                           mscale=self.position.mscale, q_temp=self.q_temp)
+                           mscale=self.position.mscale, q_temp=self.q_temp,
+                           unit_eps=self.qk_norm_eps if self.qk_norm == "unit" else None, v_mix=v_mix)
         gate = None
         if self.gate_rows:
             at = H * hd + (KVH * (hd + self.vd) if writes else 0)
@@ -444,7 +478,7 @@ class Attention(Mixer):
         if not self.values_are_keys:
             if self.qk_norm == "head":
                 ops.qk_head_norm(qk, qk, self.q_norm_w, self.k_norm_w, H, KVH, hd, self.qk_norm_eps, rows)
-            elif self.qk_norm:
+            elif self.qk_norm == "projection":
                 raise ValueError(f"{self.prefix}: a convolution goes with the heads' own norm or none")
             return qk
         out = ctx.alloc((rows, C + KVH * hd))

@@ -175,6 +175,9 @@ class StepContext:
                                           # LayerCache.page_table[seq_slot[row_seq[row]]] and skip that chain)
         self.tokens = None                # int32 [rows] the step's token ids (set by the model; a part that looks a token
                                           # up in a table of its own reads them)
+        self.room: dict = {}              # part -> rows of its own that live as long as the step (Part.step_columns)
+        self.handed: dict = {}            # what a part leaves for parts that run after it in this step, by a name of theirs
+        self.takes_pair = False           # the running mixer may return a NormedPair
         self.next_norm = None             # the norm that reads the stream after the running block (set by the model)
         self.sink = None                  # ResidualSink offered to the running mixer / feed-forward
 
@@ -230,6 +233,11 @@ class Part:
 
     def children(self) -> list["Part"]:
         return []
+
+    def step_columns(self) -> int:
+        """Columns (activation dtype) of rows this part wants to keep until the step's end, beyond its layer's turn:
+        the model then gives it ctx.room[self], [rows, columns], in every step. 0: none."""
+        return 0
 
 
 class Norm(Part):
@@ -349,6 +357,27 @@ class NormedRows:
         from ..kernels import ops
         out = ctx.alloc((self.rows, self.dim), self.scaled.dtype)
         ops.scale_rows(out, self.scaled, self.partials, self.eps, self.rows, self.pieces)
+        return out
+
+
+@dataclasses.dataclass
+class NormedPair:
+    """Two branch results whose norms and sum are still owed: rmsnorm(first) * gain_first + rmsnorm(second) *
+    gain_second, both with `eps`. Returned in place of a tensor by a mixer whose block says (ctx.takes_pair) that
+    it forms the sum on the way into the stream; tensor() gives the sum to anything else."""
+
+    first: torch.Tensor
+    second: torch.Tensor
+    gain_first: torch.Tensor
+    gain_second: torch.Tensor
+    eps: float
+    rows: int
+
+    def tensor(self, ctx: StepContext) -> torch.Tensor:
+        from ..kernels import ops
+        out = ctx.alloc((self.rows, self.first.shape[-1]), self.first.dtype)
+        ops.add_normed_pair(None, self.first, self.second, self.gain_first, self.gain_second, self.eps, 1.0, None, 0.0,
+                            None, 0.0, out, self.rows)
         return out
 
 

@@ -17,7 +17,7 @@ from __future__ import annotations
 
 import torch
 
-from .base import (Block, BuildEnv, LayerCache, PartSpec, ResidualStream, StepContext,
+from .base import (Block, BuildEnv, LayerCache, NormedPair, PartSpec, ResidualStream, StepContext,
                    build_part, param, register_part)
 
 
@@ -138,7 +138,8 @@ class SandwichNormBlock(Block):
     Every sum is one launch where the norms around it are RMS norms with a gain: the branch output
     is normed and added in fp32, and the same launch forms what the next reader wants of the new
     stream (the next pre-norm, the plain rows for the token input, or the first norm of the block
-    that follows). Other norms go through their own add_norm on a 32-bit copy of the branch output.
+    that follows); so is the sum of a mixer that hands over two branches whose norms it still owes (NormedPair). Other
+    norms go through their own add_norm on a 32-bit copy of the branch output.
 
     names: mixer_norm, mixer_post_norm, mixer, feed_forward_norm, feed_forward_post_norm,
     feed_forward, token_input (suffixes of the parts' prefixes)."""
@@ -197,9 +198,16 @@ class SandwichNormBlock(Block):
         read_c = self._rms(reader) if reader is not None and reader != "rows" else None
         if post_c is not None and (reader is None or reader == "rows" or read_c is not None):
             out = None if reader is None else ctx.alloc((rows, resid.shape[-1]))
+            if isinstance(delta, NormedPair):
+                ops.add_normed_pair(resid, delta.first, delta.second, delta.gain_first, delta.gain_second, delta.eps, 1.0,
+                                    post_c[0], post_c[1], read_c[0] if read_c else None, read_c[1] if read_c else 0.0,
+                                    out, rows)
+                return out
             ops.add_normed(resid, delta, post_c[0], post_c[1], read_c[0] if read_c else None,
                            read_c[1] if read_c else 0.0, out, rows)
             return out
+        if isinstance(delta, NormedPair):
+            delta = delta.tensor(ctx)
         # any other norm: the branch output through the norm's own kernel on a 32-bit copy, then the sum
         copy = ctx.alloc((rows, resid.shape[-1]), torch.float32)
         copy[:rows].copy_(delta[:rows])
@@ -217,7 +225,9 @@ class SandwichNormBlock(Block):
         after = ctx.next_norm                  # reads the stream once this block is done
         ctx.sink = None
         n = stream.normed(self.mixer_norm, ctx)
+        ctx.takes_pair = True
         delta = self.mixer.forward(n, ctx, cache)
+        ctx.takes_pair = False
         # who reads the stream after each sum
         tail = "rows" if self.token_input is not None else after
         n = self._join(stream, delta, self.mixer_post, self.ff_norm if self.feed_forward is not None else tail, ctx)

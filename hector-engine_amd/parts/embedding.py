@@ -5,13 +5,16 @@ stream (reference: src/graph_builder.cpp:998, kernels/linear.cu:36-69).
 Head: logits = n W^T with W the head's own matrix, or the embedding matrix when
 tied (src/graph_builder.cpp:1019-1036); only the wanted rows are computed and
 the logits are fp32 in both precisions.
+
+The embedding's `norm` (a norm that is a row scale and a gain, with its own prefix `norm_prefix`) is applied to the row
+before it becomes the stream, in the same launch.
 """
 from __future__ import annotations
 
 import torch
 
 from ..kernels import ops
-from .base import BuildEnv, Part, StepContext, TensorSpec, param, register_part, tensor_name
+from .base import BuildEnv, Part, PartSpec, StepContext, TensorSpec, build_part, param, register_part, tensor_name
 from .linear import Linear
 
 
@@ -24,16 +27,29 @@ class TokenEmbedding(Part):
         self.scale = param(params, "scale", float, 1.0)      # h[t] = E[id_t] * scale
         self._name = tensor_name(prefix, param(params, "names", dict, {}), "weight", "weight")
         self.table: torch.Tensor | None = None
+        spec = param(params, "norm", PartSpec, None)
+        self.norm = None if spec is None else build_part("norm", spec, param(params, "norm_prefix", str), env)
+
+    def children(self):
+        return [] if self.norm is None else [self.norm]
 
     def tensor_specs(self):
-        return {self._name: TensorSpec((self.vocab, self.hidden))}
+        specs = {self._name: TensorSpec((self.vocab, self.hidden))}
+        for c in self.children():
+            specs.update(c.tensor_specs())
+        return specs
 
     def bind(self, tensors):
         self.table = tensors[self._name]
+        for c in self.children():
+            c.bind(tensors)
+            if c.carried() is None or len(c.carried()) != 2:
+                raise ValueError("token_embedding: its norm must be a row scale and a gain")
 
     def forward(self, ids: torch.Tensor, rows: int, ctx: StepContext) -> torch.Tensor:
         out = ctx.alloc((rows, self.hidden), torch.float32)
-        ops.embedding(out, self.table, ids, rows, self.scale)
+        gain, eps = (None, 0.0) if self.norm is None else self.norm.carried()
+        ops.embedding(out, self.table, ids, rows, self.scale, gain, eps)
         return out
 
 

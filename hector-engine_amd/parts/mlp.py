@@ -8,7 +8,8 @@ activation "clamped_swiglu" is the same feed-forward through a bounded gate:
 g' = min(g, limit), u' = clamp(u, -limit, limit), act = g' * sigmoid(alpha * g') * (u' + 1), with
 the parameters `limit` and `alpha` (1.702 unless given). activation "gelu_tanh" has gelu's tanh form for the
 gate, 0.5 g (1 + tanh(c (g + a g^3))) with c = sqrt(2 / pi) and a = 0.044715, which is
-g * sigmoid(2 c g + 2 c a g^3). names: the suffixes of its tensors
+g * sigmoid(2 c g + 2 c a g^3). activation "relu" has max(g, 0) for the gate: g * sigmoid(alpha g) with an alpha
+so large that the sigmoid is a step. names: the suffixes of its tensors
 (gate, up, down)."""
 from __future__ import annotations
 
@@ -44,6 +45,8 @@ class GatedMLP(FeedForward):
         elif act == "gelu_tanh":
             two_c = 2.0 * math.sqrt(2.0 / math.pi)
             self.act = {"alpha": two_c, "cubic": 0.044715 * two_c}
+        elif act == "relu":
+            self.act = {"alpha": 1e30}            # the sigmoid is 0, 1/2 (at 0 alone) or 1
         else:
             raise ValueError(f"gated_mlp: unsupported activation '{act}'")
         names = param(params, "names", dict, {})

@@ -1,7 +1,10 @@
 """RMS normalisation: y = x * rsqrt(mean(x^2) + eps) * weight, the weight
 multiplying directly (reference: kernels/normalization.cu:36-63). Applied to the
 fp32 residual stream, fused with the pending residual add
-(kernels/fused_add_rmsnorm.cu:47-81)."""
+(kernels/fused_add_rmsnorm.cu:47-81).
+
+offset o (0 unless given): the stored weight is the difference from o, the gain is o + weight. scale (1 unless
+given) multiplies the result. Either is folded into the gain, which is then kept in 32-bit."""
 from __future__ import annotations
 
 import torch
@@ -16,15 +19,19 @@ class RMSNorm(Norm):
         super().__init__(prefix, env)
         self.size = param(params, "size", int)
         self.eps = param(params, "eps", float)
+        self.offset = param(params, "offset", float, 0.0)
+        self.scale = param(params, "scale", float, 1.0)
         # names: the suffix of its tensor (weight)
         self._name = tensor_name(prefix, param(params, "names", dict, {}), "weight", "weight")
         self.weight: torch.Tensor | None = None
 
     def tensor_specs(self):
-        return {self._name: TensorSpec((self.size,), ("gain", 1.0, 0.1))}
+        return {self._name: TensorSpec((self.size,), ("gain", 1.0 - self.offset, 0.1))}
 
     def bind(self, tensors):
         self.weight = tensors[self._name]
+        if self.offset != 0.0 or self.scale != 1.0:
+            self.weight = ((self.weight.float() + self.offset) * self.scale).contiguous()
 
     def carried(self):
         return self.weight, self.eps

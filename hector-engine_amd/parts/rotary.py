@@ -12,7 +12,8 @@ slow} stretches the slow frequencies for contexts longer than `original` positio
 dim(t) = r ln(original / (2 pi t)) / (2 ln theta), lo = max(floor(dim(fast)), 0),
 hi = min(ceil(dim(slow)), r - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), frequency
 i becomes f_i / factor * ramp_i + f_i (1 - ramp_i), and cos and sin are both multiplied by
-0.1 ln(factor) + 1 (`mscale`; the rotated pairs grow by that factor)."""
+0.1 ln(factor) + 1 (`mscale`; the rotated pairs grow by that factor). `scaling` = {"kind": "linear", factor}: every
+frequency is divided by factor."""
 from __future__ import annotations
 
 import math
@@ -40,8 +41,13 @@ class Rotary(PositionEncoding):
         scaling = param(params, "scaling", dict, None)
         if scaling is not None:
             kind = scaling.get("kind", "yarn")
-            if kind != "yarn":
+            if kind not in ("yarn", "linear"):
                 raise ValueError(f"rotary: unknown scaling '{kind}'")
+            if kind == "linear" and float(scaling["factor"]) <= 0:
+                raise ValueError("rotary: linear scaling needs factor > 0")
+        if scaling is not None and kind == "linear":
+            inv = inv / float(scaling["factor"])
+        elif scaling is not None:
             factor, original = float(scaling["factor"]), float(scaling["original"])
             if factor <= 0 or original <= 0 or self.theta <= 1:
                 raise ValueError("rotary: yarn scaling needs factor > 0, original > 0 and theta > 1")
