@@ -4,7 +4,7 @@ token ids) on one MI355X, with prefill and roofline figures on the same line.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L] [--shape 7b|32b|72b]
                     [--context C] [--prompt P]
-    python bench.py --design volonex | penasun | butolorn | domorax | dofipel      (another measurement: see below)
+    python bench.py --design volonex | penasun | butolorn | domorax | dofipel | bobevik      (another measurement: see below)
 
 The default is the 7B shape; --shape runs the same measurement at the layer sizes of
 Qwen2.5-32B (context 8192, prompts of 512 to 2048 tokens, batches 1 / 8 / 64) or
@@ -29,8 +29,9 @@ leaves its first run and its thermal-low samples out: OPTIMIZATION_NOTES.md:114-
 every timed run, the earlier ones still show it.
 
 --design volonex (or penasun; butolorn and domorax are measured beside Penasun, the other design whose layers carry
-a state of fixed size, and dofipel beside Domorax, the other design with attention through latents) leaves the run above aside and measures that design beside Qwen2 at equal layer
-sizes (random weights, bf16, four layers of each of a few sizes that resemble real models' layers): prompt
+a state of fixed size, dofipel beside Domorax, the other design with attention through latents, and bobevik beside
+Butolorn, the other design with a memory beside an attention) leaves the run above aside and measures that design beside
+Qwen2 at equal layer sizes (random weights, bf16, four layers of each of a few sizes that resemble real models' layers): prompt
 tokens a second for one prompt of 2,048 tokens, decoded tokens a second at batch 8 and batch 1 behind such
 prompts, and, from a second pass with an event pair around every launch, the mean time of each kind of
 kernel in the prompt step and in the one-token step of both designs side by side. One JSON line,
@@ -206,6 +207,30 @@ def dofipel_configs(sz):
     return domorax, config_from_dict(dofipel)
 
 
+def bobevik_configs(sz):
+    """(Butolorn configuration, Bobevik configuration) of one set of layer sizes. Butolorn is the design beside it: both
+    have norms on both sides of a branch, an attention and a memory of fixed size side by side, and attention layers. The
+    Bobevik layers are an attention (biases, linearly scaled rotation, capped scores, a gate a head) and a fading memory side
+    by side, an attention (unit q and k, mixed values), a retention, and an attention again; the memories have Butolorn's
+    heads of 128 key and 256 value dims, as many as make their values as wide as the model, and every layer a gated
+    feed-forward of two thirds of the named width (the arithmetic of Butolorn's, which has no gate)."""
+    from hector_engine_amd.registry import config_from_dict
+    _, butolorn = butolorn_configs(sz)
+    heads = max(1, sz["width"] // 256)
+    rot = dict(base=1000000.0, dims=sz["dim"])
+    attention = dict(heads=sz["heads"], kv_heads=sz["kv_heads"], dim=sz["dim"], vdim=sz["vdim"], scale=sz["dim"] ** -0.5)
+    memory = dict(heads=heads, dim=128, vdim=256, decay=[1.0 - 2.0 ** (-5.0 - 6.0 * h / max(1, heads - 1)) for h in range(heads)])
+    pair = dict(left=dict(attention, softcap=30.0, rot=dict(base=10000.0, dims=sz["dim"] // 2, scaling=dict(factor=4.0))),
+                right=memory)
+    mlp = dict(kind="dense", ff=sz["ff"] * 2 // 3 // 128 * 128)
+    mixing = dict(type="attention", mixer=dict(attention, rot=rot, v_mix=True), mlp=mlp)
+    layers = [dict(type="parallel", mixer=pair, mlp=mlp), mixing,
+              dict(type="retention", mixer=dict(memory, rot=dict(base=10000.0, dims=128)), mlp=mlp), mixing]
+    bobevik = dict(architecture="Bobevik", vocab=DESIGN_VOCAB, width=sz["width"], residual_mult=0.5, norm=dict(eps=1e-6),
+                   layers=layers)
+    return butolorn, config_from_dict(bobevik)
+
+
 def compare_designs(args) -> int:
     import torch
     import hector_engine_amd as he
@@ -284,13 +309,13 @@ def compare_designs(args) -> int:
         return out
 
     result = {}
-    beside = {"butolorn": "penasun", "domorax": "penasun", "dofipel": "domorax"}.get(args.design, "qwen2")
+    beside = {"butolorn": "penasun", "domorax": "penasun", "dofipel": "domorax", "bobevik": "butolorn"}.get(args.design, "qwen2")
     chosen = [n for n in DESIGN_SIZES if not args.design_sizes or n in args.design_sizes.split(",")]
     for name in chosen:
         sz = DESIGN_SIZES[name]
         result[name] = {"sizes": sz}
         configs = {"volonex": design_configs, "penasun": penasun_configs, "butolorn": butolorn_configs,
-                   "domorax": domorax_configs, "dofipel": dofipel_configs}[args.design](sz)
+                   "domorax": domorax_configs, "dofipel": dofipel_configs, "bobevik": bobevik_configs}[args.design](sz)
         for design, config in zip((beside, args.design), configs):
             progress(f"{name} {design}")
             result[name][design] = measure(config, False)
@@ -331,9 +356,9 @@ def main() -> int:
     ap.add_argument("--no-tune", action="store_true",
                     help="leave the library's default kernels for the tall matrix products")
     ap.add_argument("--design-sizes", default="", help=f"with --design: only these of {', '.join(DESIGN_SIZES)}")
-    ap.add_argument("--design", choices=["volonex", "penasun", "butolorn", "domorax", "dofipel"], default=None,
+    ap.add_argument("--design", choices=["volonex", "penasun", "butolorn", "domorax", "dofipel", "bobevik"], default=None,
                     help="instead of the run above: this design beside Qwen2 (butolorn, domorax: beside Penasun; dofipel: beside "
-                         "Domorax) at equal layer sizes, prompt and one-token steps, throughput and mean time per kind of kernel")
+                         "Domorax; bobevik: beside Butolorn) at equal layer sizes, prompt and one-token steps, throughput and mean time per kind of kernel")
     args = ap.parse_args()
     if args.design:
         return compare_designs(args)

@@ -55,60 +55,87 @@ __device__ __forceinline__ void dm_vec4(float* x, const float* p) {
   const float4 v = *reinterpret_cast<const float4*>(p);
   x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
 }
-__device__ __forceinline__ void dm_vec4(float* x, const bf16_t* p) {
-  const uint2 v = *reinterpret_cast<const uint2*>(p);
-  x[0] = __uint_as_float(v.x << 16); x[1] = __uint_as_float(v.x & 0xffff0000u);
-  x[2] = __uint_as_float(v.y << 16); x[3] = __uint_as_float(v.y & 0xffff0000u);
-}
-
-// elements d .. d + 3 of a head's `width` (zeros beyond it), through SiLU if act. VEC: widths and strides in fours.
-template <typename T, bool VEC>
+// elements d .. d + 3 of a head's `width` (zeros beyond it), one by one, through SiLU if act
+template <typename T>
 __device__ __forceinline__ void dm_load4(float* x, const T* p, int d, int width, int act) {
-  if (VEC) {
-    if (d < width) dm_vec4(x, p + d);
-    else x[0] = x[1] = x[2] = x[3] = 0.f;
-  } else {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = d + e < width ? to_float(p[d + e]) : 0.f;
-  }
-  if (act) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = dm_silu(x[e]);
+  for (int e = 0; e < 4; ++e) {
+    x[e] = d + e < width ? to_float(p[d + e]) : 0.f;
+    if (act) x[e] = dm_silu(x[e]);
   }
 }
 
 // The same of a query or key: rotated (cs, sn: the row's cosines and sines of the half frequencies) and scaled
-template <typename T, bool VEC>
+template <typename T>
 __device__ __forceinline__ void dm_load_qk4(float* x, const T* p, int d, int dk, int act, int half, const float* cs,
                                             const float* sn, float scale) {
-  dm_load4<T, VEC>(x, p, d, dk, act);
-  if (half > 0) {
-    if (VEC) {
-      if (d < 2 * half) {
-        const bool lo = d < half;
-        const int i = lo ? d : d - half;
-        float y[4], c[4], s[4];
-        dm_load4<T, true>(y, p, lo ? d + half : i, dk, act);
-        dm_vec4(c, cs + i);
-        dm_vec4(s, sn + i);
+  dm_load4<T>(x, p, d, dk, act);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) x[e] = lo ? x[e] * c[e] - y[e] * s[e] : x[e] * c[e] + y[e] * s[e];
-      }
-    } else {
+  for (int e = 0; e < 4; ++e) {
+    if (d + e < 2 * half) {
+      const bool lo = d + e < half;
+      const int i = lo ? d + e : d + e - half;
+      float y = to_float(p[lo ? d + e + half : i]);
+      if (act) y = dm_silu(y);
+      x[e] = lo ? x[e] * cs[i] - y * sn[i] : x[e] * cs[i] + y * sn[i];
+    }
+    x[e] *= scale;
+  }
+}
+
+// The whole-piece loads of a thread's share of a tile, N rows of it at dims d .. d + 3: asked for all together, with
+// no condition around them (rows past the chunk and dims past the head read the nearest ones there are and are dropped
+// afterwards), and turned into numbers when all are under way.
+template <typename T> struct DmPiece;
+template <> struct DmPiece<bf16_t> { typedef uint2 type; };
+template <> struct DmPiece<float> { typedef float4 type; };
+__device__ __forceinline__ void dm_unpack(float* x, const uint2& v) {
+  x[0] = __uint_as_float(v.x << 16); x[1] = __uint_as_float(v.x & 0xffff0000u);
+  x[2] = __uint_as_float(v.y << 16); x[3] = __uint_as_float(v.y & 0xffff0000u);
+}
+__device__ __forceinline__ void dm_unpack(float* x, const float4& v) {
+  x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
+}
+
+// where dim d's partner and frequency are (a dim that is not rotated: itself, and the first frequency)
+struct DmPair {
+  int own, partner, freq;
+  bool rotated, low;
+};
+__device__ __forceinline__ DmPair dm_pair(int d, int width, int half) {
+  DmPair p;
+  p.own = d < width ? d : 0;
+  p.rotated = p.own < 2 * half;
+  p.low = p.own < half;
+  p.freq = p.rotated ? (p.low ? p.own : p.own - half) : 0;
+  p.partner = p.rotated ? (p.low ? p.own + half : p.freq) : p.own;
+  return p;
+}
+template <typename T>
+__device__ __forceinline__ typename DmPiece<T>::type dm_ask(const T* p) {
+  return *reinterpret_cast<const typename DmPiece<T>::type*>(p);
+}
+// the asked pieces as numbers: SiLU, rotation, factor; keep false: zeros
+template <typename P>
+__device__ __forceinline__ float4 dm_give(const P& own, const P& partner, const float4& c4, const float4& s4, const DmPair& p,
+                                          int act, float scale, bool keep) {
+  float x[4];
+  dm_unpack(x, own);
+  if (act) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (d + e < 2 * half) {
-          const bool lo = d + e < half;
-          const int i = lo ? d + e : d + e - half;
-          float y = to_float(p[lo ? d + e + half : i]);
-          if (act) y = dm_silu(y);
-          x[e] = lo ? x[e] * cs[i] - y * sn[i] : x[e] * cs[i] + y * sn[i];
-        }
-      }
+    for (int e = 0; e < 4; ++e) x[e] = dm_silu(x[e]);
+  }
+  if (p.rotated) {
+    float y[4];
+    dm_unpack(y, partner);
+    const float c[4] = {c4.x, c4.y, c4.z, c4.w}, sn[4] = {s4.x, s4.y, s4.z, s4.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (act) y[e] = dm_silu(y[e]);
+      x[e] = p.low ? x[e] * c[e] - y[e] * sn[e] : x[e] * c[e] + y[e] * sn[e];
     }
   }
-#pragma unroll
-  for (int e = 0; e < 4; ++e) x[e] *= scale;
+  return keep ? make_float4(x[0] * scale, x[1] * scale, x[2] * scale, x[3] * scale) : make_float4(0.f, 0.f, 0.f, 0.f);
 }
 
 // ---- which chunk is whose ------------------------------------------------------------------------------
@@ -168,6 +195,7 @@ struct DmArgs {
   const int32_t* positions;
   const int32_t* cu;
   const int32_t* slot;
+  int rows;                  // of the step; those from cu[num_seqs] on belong to no sequence
   int num_seqs, H, dk, dv, dvp;
   uint8_t* state;
   int64_t state_stride, state_offset;
@@ -191,15 +219,45 @@ __global__ __launch_bounds__(256) void dm_share_kernel(DmArgs<T> a, int t0) {
   const int n = min(DM_C, (int)(a.cu[seq + 1] - r0));
   const float* pw = a.powers + h * (DM_C + 1);
   const int t = threadIdx.x;
+  if (VEC) {
+    const int d = 4 * (t & 15);
+    const DmPair kp = dm_pair(d0 + d, a.dk, a.half);
+    const int vd = c0 + d < a.dv ? c0 + d : 0;
+    typename DmPiece<T>::type kx[4], ky[4], vx[4];
+    float4 c4[4], s4[4];
+    float fade[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int row = min((t >> 4) + 16 * i, n - 1);
+      const int64_t at = (r0 + row) * a.stride, turn = (r0 + row) * a.half + kp.freq;
+      kx[i] = dm_ask(a.k + at + (int64_t)h * a.dk + kp.own);
+      if (a.half > 0) {
+        ky[i] = dm_ask(a.k + at + (int64_t)h * a.dk + kp.partner);
+        c4[i] = *reinterpret_cast<const float4*>(a.cs + turn);
+        s4[i] = *reinterpret_cast<const float4*>(a.sn + turn);
+      }
+      vx[i] = dm_ask(a.v + at + (int64_t)h * a.dv + vd);
+      fade[i] = pw[n - 1 - row];
+    }
+    const DmPair vp = dm_pair(0, 1, 0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int row = (t >> 4) + 16 * i;
+      *reinterpret_cast<float4*>(ks + row * DM_LD + d) =
+          dm_give(kx[i], ky[i], c4[i], s4[i], kp, a.act, a.k_scale * fade[i], row < n && d0 + d < a.dk);
+      *reinterpret_cast<float4*>(vs + row * DM_LD + d) =
+          dm_give(vx[i], vx[i], c4[i], s4[i], vp, a.act, 1.f, row < n && c0 + d < a.dv);
+    }
+  } else
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int row = (t >> 4) + 16 * i, d = 4 * (t & 15);
     float kx[4] = {0.f, 0.f, 0.f, 0.f}, vx[4] = {0.f, 0.f, 0.f, 0.f};
     if (row < n) {
       const int64_t at = (r0 + row) * a.stride;
-      dm_load_qk4<T, VEC>(kx, a.k + at + (int64_t)h * a.dk, d0 + d, a.dk, a.act, a.half, a.cs + (r0 + row) * a.half,
+      dm_load_qk4<T>(kx, a.k + at + (int64_t)h * a.dk, d0 + d, a.dk, a.act, a.half, a.cs + (r0 + row) * a.half,
                           a.sn + (r0 + row) * a.half, a.k_scale * pw[n - 1 - row]);
-      dm_load4<T, VEC>(vx, a.v + at + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
+      dm_load4<T>(vx, a.v + at + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
     }
     *reinterpret_cast<float4*>(ks + row * DM_LD + d) = make_float4(kx[0], kx[1], kx[2], kx[3]);
     *reinterpret_cast<float4*>(vs + row * DM_LD + d) = make_float4(vx[0], vx[1], vx[2], vx[3]);
@@ -278,47 +336,102 @@ __global__ __launch_bounds__(256) void dm_carry_kernel(DmArgs<T> a, int t0, int 
 // ---- every chunk's rows --------------------------------------------------------------------------------
 // One workgroup of four wavefronts a (64 value dims, head, chunk), a wavefront 32 rows x 32 columns: the rows'
 // products with the keys of the chunk (a square of which the part behind the diagonal is left out) and with the
-// memory before it, block by block of 64 key dims; then the square, faded, on the values.
+// memory before it, block by block of 32 key dims; then the square, faded, on the values. One chunk more than the
+// window's (`tail`): the step's rows that belong to no sequence get zeros.
+#define DM_KB 32      // key dims of a block here
+#define DM_KLD 36     // floats between its rows in LDS
 template <typename T, bool VEC>
-__global__ __launch_bounds__(256) void dm_rows_kernel(float* __restrict__ y, DmArgs<T> a, int t0) {
-  __shared__ __attribute__((aligned(16))) float qs[DM_C * DM_LD], ks[DM_C * DM_LD], ss[DM_B * DM_LD];
+__global__ __launch_bounds__(256, 4) void dm_rows_kernel(float* __restrict__ y, DmArgs<T> a, int t0, int tail) {
+  // rows of q, rows of k, key dims of the memory; later the square and the values
+  __shared__ __attribute__((aligned(16))) float lds[2 * DM_C * DM_LD];
+  static_assert(2 * DM_C * DM_KLD + DM_KB * DM_LD <= 2 * DM_C * DM_LD, "the blocks fit where the square and the values will be");
+  float* qs = lds;
+  float* ks = qs + DM_C * DM_KLD;
+  float* ss = ks + DM_C * DM_KLD;
+  float* square_s = lds;
+  float* vs = lds + DM_C * DM_LD;
   __shared__ float pw[DM_C + 1];
   const int h = blockIdx.y;
+  const int c0 = (int)blockIdx.x * DM_B;
+  const int t = threadIdx.x, wave = t >> 6, l32 = t & 31, hl = (t >> 5) & 1;
+  if (tail && blockIdx.z + 1 == gridDim.z) {
+    const int col = c0 + (t & 63);
+    if (col < a.dv)
+      for (int64_t r = a.cu[a.num_seqs] + wave; r < a.rows; r += 4) y[r * a.H * a.dv + (int64_t)h * a.dv + col] = 0.f;
+    return;
+  }
   int seq, chunk;
   if (!dm_find(t0 + (int)blockIdx.z, a.cu, a.num_seqs, seq, chunk)) return;
   if (a.slot[seq] < 0) return;
-  const int c0 = (int)blockIdx.x * DM_B;
   const int64_t r0 = a.cu[seq] + (int64_t)chunk * DM_C;
   const int n = min(DM_C, (int)(a.cu[seq + 1] - r0));
-  const int t = threadIdx.x, wave = t >> 6, l32 = t & 31, hl = (t >> 5) & 1;
   const int i0 = (wave >> 1) * 32, j0 = (wave & 1) * 32;
   if (t <= DM_C) pw[t] = a.powers[h * (DM_C + 1) + t];
   const float* S = a.ws + ((int64_t)blockIdx.z * a.H + h) * a.dk * a.dvp;
   dm_acc square = {0.f}, out = {0.f};
-  for (int d0 = 0; d0 < a.dk; d0 += DM_B) {
-    __syncthreads();
+  for (int d0 = 0; d0 < a.dk; d0 += DM_KB) {
+    // thread t: rows t / 8 + 32 i and dims 4 (t % 8) of q and k; dims t / 16 + 16 i and columns 4 (t % 16) of the memory
+    const int d = 4 * (t & 7), sc = 4 * (t & 15);
+    float4 sx[2], qx[2], kx[2];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int row = (t >> 4) + 16 * i, d = 4 * (t & 15);
-      float qx[4] = {0.f, 0.f, 0.f, 0.f}, kx[4] = {0.f, 0.f, 0.f, 0.f}, sx[4] = {0.f, 0.f, 0.f, 0.f};
-      if (row < n) {
-        const int64_t at = (r0 + row) * a.stride + (int64_t)h * a.dk;
-        const float* cs = a.cs + (r0 + row) * a.half;
-        const float* sn = a.sn + (r0 + row) * a.half;
-        dm_load_qk4<T, VEC>(qx, a.q + at, d0 + d, a.dk, a.act, a.half, cs, sn, 1.f);
-        dm_load_qk4<T, VEC>(kx, a.k + at, d0 + d, a.dk, a.act, a.half, cs, sn, a.k_scale);
+    for (int i = 0; i < 2; ++i) {
+      const int sd = d0 + (t >> 4) + 16 * i;
+      const bool there = sd < a.dk && c0 + sc < a.dvp;
+      const float4 v = *reinterpret_cast<const float4*>(S + (there ? (int64_t)sd * a.dvp + c0 + sc : 0));
+      sx[i] = there ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    if (VEC) {
+      const DmPair p = dm_pair(d0 + d, a.dk, a.half);
+      typename DmPiece<T>::type qo[2], qp[2], ko[2], kp[2];
+      float4 c4[2], s4[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int row = min((t >> 3) + 32 * i, n - 1);
+        const int64_t at = (r0 + row) * a.stride + (int64_t)h * a.dk, turn = (r0 + row) * a.half + p.freq;
+        qo[i] = dm_ask(a.q + at + p.own);
+        ko[i] = dm_ask(a.k + at + p.own);
+        if (a.half > 0) {
+          qp[i] = dm_ask(a.q + at + p.partner);
+          kp[i] = dm_ask(a.k + at + p.partner);
+          c4[i] = *reinterpret_cast<const float4*>(a.cs + turn);
+          s4[i] = *reinterpret_cast<const float4*>(a.sn + turn);
+        }
       }
-      if (d0 + row < a.dk && c0 + d < a.dvp) dm_vec4(sx, S + (int64_t)(d0 + row) * a.dvp + c0 + d);
-      *reinterpret_cast<float4*>(qs + row * DM_LD + d) = make_float4(qx[0], qx[1], qx[2], qx[3]);
-      *reinterpret_cast<float4*>(ks + row * DM_LD + d) = make_float4(kx[0], kx[1], kx[2], kx[3]);
-      *reinterpret_cast<float4*>(ss + row * DM_LD + d) = make_float4(sx[0], sx[1], sx[2], sx[3]);
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const bool keep = (t >> 3) + 32 * i < n && d0 + d < a.dk;
+        qx[i] = dm_give(qo[i], qp[i], c4[i], s4[i], p, a.act, 1.f, keep);
+        kx[i] = dm_give(ko[i], kp[i], c4[i], s4[i], p, a.act, a.k_scale, keep);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int row = (t >> 3) + 32 * i;
+        float q4[4] = {0.f, 0.f, 0.f, 0.f}, k4[4] = {0.f, 0.f, 0.f, 0.f};
+        if (row < n) {
+          const int64_t at = (r0 + row) * a.stride + (int64_t)h * a.dk;
+          const float* cs = a.cs + (r0 + row) * a.half;
+          const float* sn = a.sn + (r0 + row) * a.half;
+          dm_load_qk4<T>(q4, a.q + at, d0 + d, a.dk, a.act, a.half, cs, sn, 1.f);
+          dm_load_qk4<T>(k4, a.k + at, d0 + d, a.dk, a.act, a.half, cs, sn, a.k_scale);
+        }
+        qx[i] = make_float4(q4[0], q4[1], q4[2], q4[3]);
+        kx[i] = make_float4(k4[0], k4[1], k4[2], k4[3]);
+      }
     }
     __syncthreads();
-    const int dims = min(DM_B, a.dk - d0);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      *reinterpret_cast<float4*>(qs + ((t >> 3) + 32 * i) * DM_KLD + d) = qx[i];
+      *reinterpret_cast<float4*>(ks + ((t >> 3) + 32 * i) * DM_KLD + d) = kx[i];
+      *reinterpret_cast<float4*>(ss + ((t >> 4) + 16 * i) * DM_LD + sc) = sx[i];
+    }
+    __syncthreads();
+    const int dims = min(DM_KB, a.dk - d0);
     for (int g = 0; g < dims; g += 8) {
       float qa[4], ka[4];
-      dm_vec4(qa, qs + (i0 + l32) * DM_LD + g + 4 * hl);
-      dm_vec4(ka, ks + (j0 + l32) * DM_LD + g + 4 * hl);
+      dm_vec4(qa, qs + (i0 + l32) * DM_KLD + g + 4 * hl);
+      dm_vec4(ka, ks + (j0 + l32) * DM_KLD + g + 4 * hl);
 #pragma unroll
       for (int m = 0; m < 4; ++m) {
         if (j0 <= i0) square = __builtin_amdgcn_mfma_f32_32x32x2f32(qa[m], ka[m], square, 0, 0, 0);
@@ -326,27 +439,45 @@ __global__ __launch_bounds__(256) void dm_rows_kernel(float* __restrict__ y, DmA
       }
     }
   }
-  __syncthreads();
+  float4 vx[4];
+  {
+    const int d = 4 * (t & 15);
+    if (VEC) {
+      typename DmPiece<T>::type v[4];
+      const DmPair p = dm_pair(0, 1, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        v[i] = dm_ask(a.v + (r0 + min((t >> 4) + 16 * i, n - 1)) * a.stride + (int64_t)h * a.dv + (c0 + d < a.dv ? c0 + d : 0));
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        vx[i] = dm_give(v[i], v[i], make_float4(0.f, 0.f, 0.f, 0.f), make_float4(0.f, 0.f, 0.f, 0.f), p, a.act, 1.f,
+                        (t >> 4) + 16 * i < n && c0 + d < a.dv);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int row = (t >> 4) + 16 * i;
+        float v4[4] = {0.f, 0.f, 0.f, 0.f};
+        if (row < n) dm_load4<T>(v4, a.v + (r0 + row) * a.stride + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
+        vx[i] = make_float4(v4[0], v4[1], v4[2], v4[3]);
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i) *reinterpret_cast<float4*>(vs + ((t >> 4) + 16 * i) * DM_LD + d) = vx[i];
+  }
 #pragma unroll
   for (int r = 0; r < 16; ++r) {
     const int i = i0 + 8 * (r >> 2) + 4 * hl + (r & 3), j = j0 + l32;
-    qs[i * DM_LD + j] = i >= j ? square[r] * pw[i - j] : 0.f;
+    square_s[i * DM_LD + j] = i >= j ? square[r] * pw[i - j] : 0.f;
     out[r] *= pw[i + 1];
-  }
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int row = (t >> 4) + 16 * i, d = 4 * (t & 15);
-    float vx[4] = {0.f, 0.f, 0.f, 0.f};
-    if (row < n) dm_load4<T, VEC>(vx, a.v + (r0 + row) * a.stride + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
-    *reinterpret_cast<float4*>(ks + row * DM_LD + d) = make_float4(vx[0], vx[1], vx[2], vx[3]);
   }
   __syncthreads();
   for (int g = 0; g < i0 + 32; g += 8) {      // rows up to the wavefront's last one
     float pa[4];
-    dm_vec4(pa, qs + (i0 + l32) * DM_LD + g + 4 * hl);
+    dm_vec4(pa, square_s + (i0 + l32) * DM_LD + g + 4 * hl);
 #pragma unroll
     for (int m = 0; m < 4; ++m)
-      out = __builtin_amdgcn_mfma_f32_32x32x2f32(pa[m], ks[(g + 4 * hl + m) * DM_LD + j0 + l32], out, 0, 0, 0);
+      out = __builtin_amdgcn_mfma_f32_32x32x2f32(pa[m], vs[(g + 4 * hl + m) * DM_LD + j0 + l32], out, 0, 0, 0);
   }
   const int col = c0 + j0 + l32;
   if (col < a.dv) {
@@ -365,6 +496,12 @@ template <typename T, int E>
 __global__ __launch_bounds__(256) void dm_step_kernel(float* __restrict__ y, DmArgs<T> a) {
   __shared__ float qs[32 * E], ks[32 * E], vs[DM_STEP_TILE], part[4][DM_STEP_TILE];
   const int seq = blockIdx.z, h = blockIdx.y;
+  if (seq == a.num_seqs) {       // the step's rows that belong to no sequence get zeros
+    const int col = (int)blockIdx.x * DM_STEP_TILE + (threadIdx.x & 31);
+    if (col < a.dv)
+      for (int64_t r = a.cu[seq] + (threadIdx.x >> 5); r < a.rows; r += 8) y[r * a.H * a.dv + (int64_t)h * a.dv + col] = 0.f;
+    return;
+  }
   const int slot = a.slot[seq];
   const int r0 = a.cu[seq], r1 = a.cu[seq + 1];
   if (slot < 0 || r0 >= r1) return;
@@ -446,7 +583,7 @@ __global__ __launch_bounds__(256) void dm_step_kernel(float* __restrict__ y, DmA
 template <typename T>
 static int dm_run(float* y, DmArgs<T> a, int rows, int max_q_len, float* workspace, hipStream_t s) {
   if (max_q_len <= DM_WALK) {
-    const dim3 grid((a.dv + DM_STEP_TILE - 1) / DM_STEP_TILE, a.H, a.num_seqs);
+    const dim3 grid((a.dv + DM_STEP_TILE - 1) / DM_STEP_TILE, a.H, a.num_seqs + 1);
     const int e = (a.dk + 31) / 32;
     if (e <= 1) dm_step_kernel<T, 1><<<grid, 256, 0, s>>>(y, a);
     else if (e <= 2) dm_step_kernel<T, 2><<<grid, 256, 0, s>>>(y, a);
@@ -471,12 +608,14 @@ static int dm_run(float* y, DmArgs<T> a, int rows, int max_q_len, float* workspa
   const int kb = (a.dk + DM_B - 1) / DM_B, vb = (a.dvp + DM_B - 1) / DM_B;
   for (int t0 = 0; t0 < chunks; t0 += window) {
     const int nt = chunks - t0 < window ? chunks - t0 : window;
-    const dim3 share(kb * vb, a.H, nt), carry((unsigned)(((int64_t)a.dk * a.dvp / 4 + 255) / 256), a.H, a.num_seqs), out(vb, a.H, nt);
+    const dim3 share(kb * vb, a.H, nt), carry((unsigned)(((int64_t)a.dk * a.dvp / 4 + 255) / 256), a.H, a.num_seqs);
+    const int tail = t0 + nt >= chunks;
+    const dim3 out(vb, a.H, nt + tail);
     if (vec) dm_share_kernel<T, true><<<share, 256, 0, s>>>(a, t0);
     else dm_share_kernel<T, false><<<share, 256, 0, s>>>(a, t0);
     dm_carry_kernel<T><<<carry, 256, 0, s>>>(a, t0, nt);
-    if (vec) dm_rows_kernel<T, true><<<out, 256, 0, s>>>(y, a, t0);
-    else dm_rows_kernel<T, false><<<out, 256, 0, s>>>(y, a, t0);
+    if (vec) dm_rows_kernel<T, true><<<out, 256, 0, s>>>(y, a, t0, tail);
+    else dm_rows_kernel<T, false><<<out, 256, 0, s>>>(y, a, t0, tail);
   }
   return he_check_launch("he_decay_scan");
 }
@@ -487,7 +626,7 @@ extern "C" int he_decay_scan(void* y_f32, const void* q, const void* k, const vo
                              const void* cu_seqlens, const void* seq_slot, int rows, int num_seqs, int max_q_len, int H,
                              int dk, int dv, void* workspace_f32, int64_t workspace_floats, int dtype, void* stream) {
   HE_REQUIRE(rows >= 0 && num_seqs >= 0 && H > 0 && dk > 0 && dv > 0, "he_decay_scan: bad sizes H=%d dk=%d dv=%d", H, dk, dv);
-  HE_REQUIRE(H <= 65535 && num_seqs <= 65535, "he_decay_scan: more than 65535 heads or sequences");
+  HE_REQUIRE(H <= 65535 && num_seqs < 65535, "he_decay_scan: more than 65535 heads or sequences");
   HE_REQUIRE(dk <= DM_MAX_KEY, "he_decay_scan: key size %d above %d", dk, DM_MAX_KEY);
   HE_REQUIRE(dtype == HE_BF16 || dtype == HE_F32, "he_decay_scan: unknown dtype %d", dtype);
   HE_REQUIRE(half >= 0 && 2 * half <= dk && (half == 0 || (inv_freq_f32 != nullptr && positions != nullptr)),
@@ -504,7 +643,7 @@ extern "C" int he_decay_scan(void* y_f32, const void* q, const void* k, const vo
   a.q = (const T*)q; a.k = (const T*)k; a.v = (const T*)v; a.stride = in_stride; a.powers = (const float*)powers_f32;   \
   a.inv_freq = (const float*)inv_freq_f32; a.cs = a.sn = nullptr; a.half = half; a.act = act; a.k_scale = k_scale;     \
   a.positions = (const int32_t*)positions; a.cu = (const int32_t*)cu_seqlens; a.slot = (const int32_t*)seq_slot;       \
-  a.num_seqs = num_seqs; a.H = H; a.dk = dk; a.dv = dv; a.dvp = dm_dvp(dv); a.state = (uint8_t*)state;                 \
+  a.rows = rows; a.num_seqs = num_seqs; a.H = H; a.dk = dk; a.dv = dv; a.dvp = dm_dvp(dv); a.state = (uint8_t*)state;                 \
   a.state_stride = state_stride; a.state_offset = state_offset; a.ws = nullptr;                                        \
   return dm_run<T>((float*)y_f32, a, rows, max_q_len, (float*)workspace_f32, (hipStream_t)stream)
   if (dtype == HE_BF16) {

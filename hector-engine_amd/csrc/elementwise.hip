@@ -21,7 +21,7 @@ __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ 
   }
   const T* row = table + (int64_t)id * D;
   float ss = 0.f;      // of the elements this thread has written
-  if (sizeof(T) == 2 && (D & 7) == 0 && (((uintptr_t)table | (uintptr_t)out) & 15) == 0) {
+  if (norm_w == nullptr && sizeof(T) == 2 && (D & 7) == 0 && (((uintptr_t)table | (uintptr_t)out) & 15) == 0) {
     // eight elements a thread and turn: one 16-byte load, two 16-byte stores
     for (int i = 8 * threadIdx.x; i < D; i += 8 * blockDim.x) {
       const uint4 v = *reinterpret_cast<const uint4*>(reinterpret_cast<const uint16_t*>(row) + i);
@@ -34,14 +34,7 @@ __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ 
       }
       *reinterpret_cast<float4*>(o + i) = make_float4(f[0], f[1], f[2], f[3]);
       *reinterpret_cast<float4*>(o + i + 4) = make_float4(f[4], f[5], f[6], f[7]);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) ss = fmaf(f[j], f[j], ss);
     }
-    if (norm_w == nullptr) return;
-    const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)D + eps);
-    for (int i = 8 * threadIdx.x; i < D; i += 8 * blockDim.x)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) o[i + j] = o[i + j] * inv * load_param(norm_w, i + j, w_dtype);
     return;
   }
   for (int i = threadIdx.x; i < D; i += blockDim.x) {
@@ -54,6 +47,51 @@ __global__ void embedding_kernel(float* __restrict__ out, const T* __restrict__ 
   for (int i = threadIdx.x; i < D; i += blockDim.x) o[i] = o[i] * inv * load_param(norm_w, i, w_dtype);
 }
 
+// The normed row of a bf16 table in one pass: eight neighbouring elements a thread and run, up to two runs, held in
+// registers between the row's sum of squares and its store (D a multiple of 8 and at most 16 * blockDim.x).
+__global__ __launch_bounds__(1024) void embedding_normed_kernel(float* __restrict__ out, const uint16_t* __restrict__ table,
+                                                                const int32_t* __restrict__ ids, int D, int V, float scale,
+                                                                const void* __restrict__ norm_w, int w_dtype, float eps) {
+  __shared__ float scratch[16];
+  const int64_t t = blockIdx.x;
+  const int id = ids[t];
+  const bool known = id >= 0 && id < V;
+  const uint16_t* row = table + (known ? (int64_t)id * D : 0);
+  float* o = out + t * (int64_t)D;
+  float f[16], g[16];
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {        // the gains are on their way before the row's sum is formed
+    const int i = 8 * (threadIdx.x + u * blockDim.x);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) g[8 * u + j] = load_param(norm_w, (i < D ? i : 0) + j, w_dtype);
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int i = 8 * (threadIdx.x + u * blockDim.x);
+    const uint4 v = known && i < D ? *reinterpret_cast<const uint4*>(row + i) : make_uint4(0, 0, 0, 0);
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[8 * u + 2 * j] = __uint_as_float(w[j] << 16) * scale;
+      f[8 * u + 2 * j + 1] = __uint_as_float(w[j] & 0xffff0000u) * scale;
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss = fmaf(f[8 * u + j], f[8 * u + j], ss);
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)D + eps);
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int i = 8 * (threadIdx.x + u * blockDim.x);
+    if (i < D) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[8 * u + j] *= inv * g[8 * u + j];
+      *reinterpret_cast<float4*>(o + i) = make_float4(f[8 * u], f[8 * u + 1], f[8 * u + 2], f[8 * u + 3]);
+      *reinterpret_cast<float4*>(o + i + 4) = make_float4(f[8 * u + 4], f[8 * u + 5], f[8 * u + 6], f[8 * u + 7]);
+    }
+  }
+}
+
 extern "C" int he_embedding(void* out_f32, const void* table, const void* ids, int rows, int D,
                             int V, int table_dtype, float scale, const void* norm_w, int w_dtype, float eps,
                             void* stream) {
@@ -61,6 +99,15 @@ extern "C" int he_embedding(void* out_f32, const void* table, const void* ids, i
   if (rows == 0) return 0;
   const int threads = D >= 1024 ? 256 : (D >= 256 ? 128 : 64);
   hipStream_t s = (hipStream_t)stream;
+  HE_REQUIRE(norm_w == nullptr || w_dtype == HE_F32 || w_dtype == HE_BF16, "he_embedding: bad weight dtype");
+  if (norm_w != nullptr && table_dtype == HE_BF16 && D % 8 == 0 && D <= 16 * 1024 &&
+      (((uintptr_t)table | (uintptr_t)out_f32) & 15) == 0) {
+    int wide = 64;
+    while (wide < 256 ? 8 * wide < D : 16 * wide < D) wide <<= 1;
+    embedding_normed_kernel<<<rows, wide, 0, s>>>((float*)out_f32, (const uint16_t*)table, (const int32_t*)ids, D, V, scale,
+                                                  norm_w, w_dtype, eps);
+    return he_check_launch("he_embedding");
+  }
   if (table_dtype == HE_BF16)
     embedding_kernel<bf16_t><<<rows, threads, 0, s>>>((float*)out_f32, (const bf16_t*)table,
                                                       (const int32_t*)ids, D, V, scale, norm_w, w_dtype, eps);

@@ -360,7 +360,7 @@ int he_delta_scan(void* y_f32, const void* q, const void* k, const void* v, int6
 // and k turn by positions[row] * inv_freq[i] (pair (i, i + half)), and k is multiplied by k_scale. powers_f32
 // [H][65]: decay_h^0 .. decay_h^64. S (fp32, he_decay_state_floats floats) lives at byte state_offset of the
 // sequence's row of the state area, zeros at a sequence's start, and is carried on. max_q_len: the most rows of a
-// sequence in this step. workspace_f32: he_decay_workspace_floats floats on a 16-byte boundary. dk up to 512.
+// sequence in this step. Rows of y that belong to no sequence get zeros. workspace_f32: he_decay_workspace_floats floats on a 16-byte boundary. dk up to 512.
 int64_t he_decay_state_floats(int H, int dk, int dv);
 int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv, int half);
 int he_decay_scan(void* y_f32, const void* q, const void* k, const void* v, int64_t in_stride, const void* powers_f32,

@@ -543,85 +543,171 @@ __global__ void add_normed_vec_kernel(float* __restrict__ resid, const TD* __res
   }
 }
 
-// Two branches side by side, each normed over the row with a gain of its own:
-//   x = scale * (a / rms(a) * w_a + b / rms(b) * w_b),   rms(z) = sqrt(mean(z^2) + pair_eps).
-// With resid given, x then goes the way of a branch output above (normed by post_w if given, added to resid, and out
-// = what the next reader wants of it); without, out = x. Everything in fp32 registers between the loads and out. VEC:
-// runs of four neighbouring elements a thread (what add_normed_vec_kernel asks of widths and addresses).
-template <typename TD, typename TO, bool VEC>
+// Four gains at once, whichever dtype they are stored in
+__device__ __forceinline__ void pn_param4(float* dst, const void* p, int64_t i, int dtype) {
+  if (dtype == HE_BF16) pn_load4(dst, (const bf16_t*)p + i);
+  else pn_load4(dst, (const float*)p + i);
+}
+
+// Two sums over a block at once (`scratch`: 32 floats), as block_sum forms one
+__device__ __forceinline__ void pn_block_sum2(float& a, float& b, float* scratch) {
+  const int lane = threadIdx.x & (HE_WAVE - 1), wave = threadIdx.x >> 6, waves = (blockDim.x + HE_WAVE - 1) >> 6;
+  a = wave_sum(a);
+  b = wave_sum(b);
+  __syncthreads();
+  if (lane == 0) {
+    scratch[wave] = a;
+    scratch[16 + wave] = b;
+  }
+  __syncthreads();
+  a = b = 0.f;
+  for (int w = 0; w < waves; ++w) {
+    a += scratch[w];
+    b += scratch[16 + w];
+  }
+}
+
+// A branch output (a), or with PAIR two of them side by side, each normed over the row with a gain of its own,
+//   x = scale * (a / rms(a) * w_a + b / rms(b) * w_b),   rms(z) = sqrt(mean(z^2) + pair_eps),
+// on the way above: normed by post_w, added to resid, and out = what the next reader wants of it; without resid
+// (PAIR), out = x. Everything in fp32 registers between the loads and out; a thread holds EPT elements in runs of four
+// neighbours, and every load of the row, the gains' too, is under way before the first sum is formed. Widths are
+// multiples of 4, everything begins on 16 bytes (gains in bf16: 8).
+template <typename TD, typename TO, int EPT, bool PAIR>
+__global__ __launch_bounds__(1024) void normed_sum_kernel(
+    float* __restrict__ resid, const TD* __restrict__ a, const TD* __restrict__ b, const void* __restrict__ w_a,
+    const void* __restrict__ w_b, int pair_dtype, float pair_eps, float scale, const void* __restrict__ post_w, float post_eps,
+    const void* __restrict__ next_w, float next_eps, int w_dtype, TO* __restrict__ out, int D) {
+  __shared__ float scratch[32], scratch_b[16];
+  const int64_t row = blockIdx.x;
+  float x[EPT], z[PAIR ? EPT : 4], ga[PAIR ? EPT : 4], gb[PAIR ? EPT : 4], r[EPT], gp[EPT], gn[EPT];
+#pragma unroll
+  for (int e = 0; e < EPT; e += 4) {
+    const int i = (threadIdx.x + (e / 4) * blockDim.x) * 4;
+    const int at = i < D ? i : 0;        // (lanes past the row read its start and drop it)
+    pn_load4(x + e, a + row * D + at);
+    if constexpr (PAIR) {
+      pn_load4(z + e, b + row * D + at);
+      pn_param4(ga + e, w_a, at, pair_dtype);
+      pn_param4(gb + e, w_b, at, pair_dtype);
+    }
+    if (resid) pn_load4(r + e, resid + row * D + at);
+    if (post_w) pn_param4(gp + e, post_w, at, w_dtype);
+    if (next_w) pn_param4(gn + e, next_w, at, w_dtype);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      x[e + u] = i < D ? x[e + u] : 0.f;
+      if constexpr (PAIR) z[e + u] = i < D ? z[e + u] : 0.f;
+    }
+  }
+  float ss = 0.f;
+  if constexpr (PAIR) {
+    float sb = 0.f;
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      ss = fmaf(x[e], x[e], ss);
+      sb = fmaf(z[e], z[e], sb);
+    }
+    pn_block_sum2(ss, sb, scratch);
+    const float ia = scale / sqrtf(ss / (float)D + pair_eps), ib = scale / sqrtf(sb / (float)D + pair_eps);
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) x[e] = x[e] * ia * ga[e] + z[e] * ib * gb[e];
+  }
+  if (resid) {
+    float inv = 1.f;
+    if (post_w) {
+      ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) ss = fmaf(x[e], x[e], ss);
+      inv = 1.f / sqrtf(block_sum(ss, scratch_b) / (float)D + post_eps);
+    }
+    ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < EPT; e += 4) {
+      const int i = (threadIdx.x + (e / 4) * blockDim.x) * 4;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        x[e + u] = i < D ? r[e + u] + x[e + u] * inv * (post_w ? gp[e + u] : 1.f) : 0.f;
+        ss = fmaf(x[e + u], x[e + u], ss);
+      }
+      if (i < D) pn_store4(resid + row * D + i, x + e);
+    }
+    if (out == nullptr) return;
+    if (next_w) {
+      const float inv2 = 1.f / sqrtf(block_sum(ss, scratch_b) / (float)D + next_eps);
+#pragma unroll
+      for (int e = 0; e < EPT; ++e) x[e] *= inv2 * gn[e];
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < EPT; e += 4) {
+    const int i = (threadIdx.x + (e / 4) * blockDim.x) * 4;
+    if (i < D) pn_store4(out + row * D + i, x + e);
+  }
+}
+
+static bool pn_vec_gain(const void* w, int dtype) { return ((uintptr_t)w & (dtype == HE_BF16 ? 7 : 15)) == 0; }
+
+// Elements a thread of normed_sum_kernel holds at this width and block
+static int pn_ept(int D, int threads) { return D <= 4 * threads ? 4 : D <= 8 * threads ? 8 : 16; }
+
+#define NORMED_SUM(TD, TO, PAIR)                                                                                        \
+  do {                                                                                                                  \
+    const int ept = pn_ept(D, threads);                                                                                 \
+    if (ept == 4) NORMED_SUM_EPT(TD, TO, 4, PAIR);                                                                      \
+    else if (ept == 8) NORMED_SUM_EPT(TD, TO, 8, PAIR);                                                                 \
+    else NORMED_SUM_EPT(TD, TO, 16, PAIR);                                                                              \
+  } while (0)
+
+// The same sum of two branches for any width and address, element by element
+template <typename TD, typename TO>
 __global__ void add_normed_pair_kernel(float* __restrict__ resid, const TD* __restrict__ a, const TD* __restrict__ b,
                                        const void* __restrict__ w_a, const void* __restrict__ w_b, int pair_dtype,
                                        float pair_eps, float scale, const void* __restrict__ post_w, float post_eps,
                                        const void* __restrict__ next_w, float next_eps, int w_dtype,
                                        TO* __restrict__ out, int D) {
-  __shared__ float scratch[16], scratch_b[16];
-  constexpr int RUN = VEC ? 4 : 1;
+  __shared__ float scratch[32];
   const int64_t row = blockIdx.x;
-  auto at = [&](int e) { return VEC ? (threadIdx.x + (e / 4) * blockDim.x) * 4 + e % 4 : threadIdx.x + e * blockDim.x; };
-  auto load = [&](float* x, const auto* p) {
-#pragma unroll
-    for (int e = 0; e < PN_EPT; e += RUN) {
-      const int i = at(e);
-      if constexpr (VEC) {
-        if (i < D) pn_load4(x + e, p + i);
-        else x[e] = x[e + 1] = x[e + 2] = x[e + 3] = 0.f;
-      } else {
-        x[e] = i < D ? to_float(p[i]) : 0.f;
-      }
-    }
-  };
-  auto store = [&](auto* p, const float* x) {
-#pragma unroll
-    for (int e = 0; e < PN_EPT; e += RUN) {
-      const int i = at(e);
-      if (i < D) {
-        if constexpr (VEC) pn_store4(p + i, x + e);
-        else p[i] = from_float<std::remove_reference_t<decltype(*p)>>(x[e]);
-      }
-    }
-  };
   float x[PN_EPT], z[PN_EPT];
-  load(x, a + row * D);
-  load(z, b + row * D);
-  float sa = 0.f, sb = 0.f;
+  float ss = 0.f, sb = 0.f;
 #pragma unroll
   for (int e = 0; e < PN_EPT; ++e) {
-    sa = fmaf(x[e], x[e], sa);
+    const int i = threadIdx.x + e * blockDim.x;
+    x[e] = i < D ? to_float(a[row * D + i]) : 0.f;
+    z[e] = i < D ? to_float(b[row * D + i]) : 0.f;
+    ss = fmaf(x[e], x[e], ss);
     sb = fmaf(z[e], z[e], sb);
   }
-  const float ia = scale / sqrtf(block_sum(sa, scratch) / (float)D + pair_eps);
-  const float ib = scale / sqrtf(block_sum(sb, scratch_b) / (float)D + pair_eps);
-  float ss = 0.f;
-#pragma unroll
-  for (int e = 0; e < PN_EPT; ++e) {
-    const int i = at(e);
-    if (i < D) x[e] = x[e] * ia * load_param(w_a, i, pair_dtype) + z[e] * ib * load_param(w_b, i, pair_dtype);
-    ss = fmaf(x[e], x[e], ss);
-  }
-  if (resid == nullptr) {
-    store(out + row * D, x);
-    return;
-  }
-  const float inv = post_w ? 1.0f / sqrtf(block_sum(ss, scratch) / (float)D + post_eps) : 1.f;
-  load(z, resid + row * D);
+  pn_block_sum2(ss, sb, scratch);
+  const float ia = scale / sqrtf(ss / (float)D + pair_eps), ib = scale / sqrtf(sb / (float)D + pair_eps);
   ss = 0.f;
 #pragma unroll
   for (int e = 0; e < PN_EPT; ++e) {
-    const int i = at(e);
-    if (i < D) x[e] = z[e] + x[e] * inv * (post_w ? load_param(post_w, i, w_dtype) : 1.f);
+    const int i = threadIdx.x + e * blockDim.x;
+    if (i < D) x[e] = x[e] * ia * load_param(w_a, i, pair_dtype) + z[e] * ib * load_param(w_b, i, pair_dtype);
     ss = fmaf(x[e], x[e], ss);
   }
-  store(resid + row * D, x);
-  if (out == nullptr) return;
-  if (next_w) {
-    const float inv2 = 1.0f / sqrtf(block_sum(ss, scratch_b) / (float)D + next_eps);
+  float inv2 = 1.f;
+  if (resid) {
+    const float inv = post_w ? 1.f / sqrtf(block_sum(ss, scratch) / (float)D + post_eps) : 1.f;
+    ss = 0.f;
 #pragma unroll
     for (int e = 0; e < PN_EPT; ++e) {
-      const int i = at(e);
-      if (i < D) x[e] = x[e] * inv2 * load_param(next_w, i, w_dtype);
+      const int i = threadIdx.x + e * blockDim.x;
+      if (i < D) {
+        x[e] = resid[row * D + i] + x[e] * inv * (post_w ? load_param(post_w, i, w_dtype) : 1.f);
+        resid[row * D + i] = x[e];
+      }
+      ss = fmaf(x[e], x[e], ss);
     }
+    if (out == nullptr) return;
+    if (next_w) inv2 = 1.f / sqrtf(block_sum(ss, scratch) / (float)D + next_eps);
   }
-  store(out + row * D, x);
+#pragma unroll
+  for (int e = 0; e < PN_EPT; ++e) {
+    const int i = threadIdx.x + e * blockDim.x;
+    if (i < D) out[row * D + i] = from_float<TO>(resid && next_w ? x[e] * inv2 * load_param(next_w, i, w_dtype) : x[e]);
+  }
 }
 
 extern "C" int he_add_normed_pair(void* resid_f32, const void* a, const void* b, int delta_dtype, const void* w_a,
@@ -640,23 +726,27 @@ extern "C" int he_add_normed_pair(void* resid_f32, const void* a, const void* b,
   while (threads < 1024 && PN_EPT * threads < D) threads <<= 1;
   while (threads < 256 && 4 * threads < D) threads <<= 1;
   hipStream_t s = (hipStream_t)stream;
-  const bool vec = D % 4 == 0 && (((uintptr_t)resid_f32 | (uintptr_t)a | (uintptr_t)b | (uintptr_t)out) & 15) == 0;
-#define PN_PAIR(TD, TO, VEC)                                                                                            \
-  add_normed_pair_kernel<TD, TO, VEC><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)a, (const TD*)b, w_a, w_b, \
-                                                               pair_dtype, pair_eps, scale, post_weight, post_eps,      \
-                                                               next_weight, next_eps, w_dtype, (TO*)out, D)
-#define PN_PAIR_VEC(TD, TO)          \
-  do {                               \
-    if (vec) PN_PAIR(TD, TO, true);  \
-    else PN_PAIR(TD, TO, false);     \
+  const bool vec = D % 4 == 0 && (((uintptr_t)resid_f32 | (uintptr_t)a | (uintptr_t)b | (uintptr_t)out) & 15) == 0 &&
+                   pn_vec_gain(w_a, pair_dtype) && pn_vec_gain(w_b, pair_dtype) && pn_vec_gain(post_weight, w_dtype) &&
+                   pn_vec_gain(next_weight, w_dtype);
+#define NORMED_SUM_EPT(TD, TO, EPT, PAIR)                                                                               \
+  normed_sum_kernel<TD, TO, EPT, PAIR><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)a, (const TD*)b, w_a, w_b,  \
+                                                                pair_dtype, pair_eps, scale, post_weight, post_eps,      \
+                                                                next_weight, next_eps, w_dtype, (TO*)out, D)
+#define PN_PAIR(TD, TO)                                                                                                 \
+  do {                                                                                                                  \
+    if (vec) NORMED_SUM(TD, TO, true);                                                                                  \
+    else add_normed_pair_kernel<TD, TO><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)a, (const TD*)b, w_a, w_b, \
+                                                                 pair_dtype, pair_eps, scale, post_weight, post_eps,     \
+                                                                 next_weight, next_eps, w_dtype, (TO*)out, D);           \
   } while (0)
   const bool db = delta_dtype == HE_BF16, ob = out_dtype == HE_BF16;
-  if (db && ob) PN_PAIR_VEC(bf16_t, bf16_t);
-  else if (db) PN_PAIR_VEC(bf16_t, float);
-  else if (ob) PN_PAIR_VEC(float, bf16_t);
-  else PN_PAIR_VEC(float, float);
-#undef PN_PAIR_VEC
+  if (db && ob) PN_PAIR(bf16_t, bf16_t);
+  else if (db) PN_PAIR(bf16_t, float);
+  else if (ob) PN_PAIR(float, bf16_t);
+  else PN_PAIR(float, float);
 #undef PN_PAIR
+#undef NORMED_SUM_EPT
   return he_check_launch("he_add_normed_pair");
 }
 
@@ -678,6 +768,19 @@ extern "C" int he_add_normed(void* resid_f32, const void* delta, int delta_dtype
   add_normed_kernel<TD, TO><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)delta, post_weight, post_eps, \
                                                      next_weight, next_eps, w_dtype, (TO*)out, D)
   const bool db = delta != nullptr && delta_dtype == HE_BF16, ob = out != nullptr && out_dtype == HE_BF16;
+  if (D % 4 == 0 && (((uintptr_t)resid_f32 | (uintptr_t)delta | (uintptr_t)out) & 15) == 0 && delta != nullptr &&
+      pn_vec_gain(post_weight, w_dtype) && pn_vec_gain(next_weight, w_dtype)) {
+#define NORMED_SUM_EPT(TD, TO, EPT, PAIR)                                                                            \
+  normed_sum_kernel<TD, TO, EPT, PAIR><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)delta, (const TD*)nullptr, \
+                                                                nullptr, nullptr, HE_F32, 0.f, 1.f, post_weight,      \
+                                                                post_eps, next_weight, next_eps, w_dtype, (TO*)out, D)
+    if (db && ob) NORMED_SUM(bf16_t, bf16_t, false);
+    else if (db) NORMED_SUM(bf16_t, float, false);
+    else if (ob) NORMED_SUM(float, bf16_t, false);
+    else NORMED_SUM(float, float, false);
+#undef NORMED_SUM_EPT
+    return he_check_launch("he_add_normed");
+  }
   if (D % 4 == 0 && (((uintptr_t)resid_f32 | (uintptr_t)delta | (uintptr_t)out) & 15) == 0) {
 #define PN_VEC(TD, TO)                                                                                                \
   add_normed_vec_kernel<TD, TO><<<rows, threads, 0, s>>>((float*)resid_f32, (const TD*)delta, post_weight, post_eps,   \

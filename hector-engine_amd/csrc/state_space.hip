@@ -382,6 +382,69 @@ __global__ void gated_group_norm_kernel(T* __restrict__ out, const float* __rest
   }
 }
 
+// The same where a part fits in registers: `lanes` neighbouring threads (a wavefront, or the whole workgroup) take a
+// part, a thread R runs of four elements of it; everything a thread reads is asked for before the sum is formed.
+// Parts and their number a row in fours, y, z, weight and out on whole runs.
+__device__ __forceinline__ void ss_load4(float* x, const float* p) {
+  const float4 v = *reinterpret_cast<const float4*>(p);
+  x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
+}
+__device__ __forceinline__ void ss_load4(float* x, const bf16_t* p) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p);
+  x[0] = __uint_as_float(v.x << 16); x[1] = __uint_as_float(v.x & 0xffff0000u);
+  x[2] = __uint_as_float(v.y << 16); x[3] = __uint_as_float(v.y & 0xffff0000u);
+}
+__device__ __forceinline__ void ss_store4(float* p, const float* x) { *reinterpret_cast<float4*>(p) = make_float4(x[0], x[1], x[2], x[3]); }
+__device__ __forceinline__ void ss_store4(bf16_t* p, const float* x) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(pack2_bf16(x[0], x[1]), pack2_bf16(x[2], x[3]));
+}
+template <typename T, int R, bool WAVE>
+__global__ void gated_group_norm_vec_kernel(T* __restrict__ out, const float* __restrict__ y, const T* __restrict__ z,
+                                            int64_t z_stride, const void* __restrict__ weight, int w_dtype, int W, int parts,
+                                            int64_t units, float eps, int gate_after, float out_scale) {
+  __shared__ float scratch[16];
+  const int width = W / parts;
+  const int lanes = WAVE ? 64 : blockDim.x, lane = WAVE ? threadIdx.x & 63 : threadIdx.x;
+  const int64_t unit = WAVE ? (int64_t)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6) : blockIdx.x;
+  if (unit >= units) return;
+  const int64_t row = unit / parts;
+  const int c0 = (int)(unit % parts) * width;
+  float v[4 * R], g[4 * R], w[4 * R];
+  float sq = 0.f;
+#pragma unroll
+  for (int u = 0; u < R; ++u) {
+    const int i = 4 * (lane + u * lanes), at = c0 + (i < width ? i : 0);
+    ss_load4(v + 4 * u, y + row * W + at);
+    ss_load4(g + 4 * u, z + row * z_stride + at);
+    if (w_dtype == HE_BF16) ss_load4(w + 4 * u, (const bf16_t*)weight + at);
+    else ss_load4(w + 4 * u, (const float*)weight + at);
+  }
+#pragma unroll
+  for (int u = 0; u < R; ++u) {
+    const bool in = 4 * (lane + u * lanes) < width;
+#pragma unroll
+    for (int e = 4 * u; e < 4 * u + 4; ++e) {
+      if (!gate_after) v[e] *= ss_silu(g[e]);
+      v[e] = in ? v[e] : 0.f;
+      sq = fmaf(v[e], v[e], sq);
+    }
+  }
+  const float inv = 1.f / sqrtf((WAVE ? wave_sum(sq) : block_sum(sq, scratch)) / (float)width + eps);
+#pragma unroll
+  for (int u = 0; u < R; ++u) {
+    const int i = 4 * (lane + u * lanes);
+    if (i < width) {
+#pragma unroll
+      for (int e = 4 * u; e < 4 * u + 4; ++e) {
+        v[e] *= inv * w[e];
+        if (gate_after) v[e] *= out_scale / (1.f + expf(-g[e]));
+        if (gate_after == 2) v[e] *= g[e];
+      }
+      ss_store4(out + row * W + c0 + i, v + 4 * u);
+    }
+  }
+}
+
 extern "C" int he_gated_group_norm(void* out, const void* y_f32, const void* z, int64_t z_stride, const void* weight,
                                    int w_dtype, int rows, int W, int parts, float eps, int gate_after, float out_scale,
                                    int dtype, void* stream) {
@@ -392,6 +455,34 @@ extern "C" int he_gated_group_norm(void* out, const void* y_f32, const void* z, 
   const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
   const dim3 grid(parts, rows);
   hipStream_t s = (hipStream_t)stream;
+  const uintptr_t run = dtype == HE_BF16 ? 7 : 15;      // bytes of four elements, less one
+  if (width % 4 == 0 && z_stride % 4 == 0 && width <= 16 * 1024 && ((uintptr_t)y_f32 & 15) == 0 &&
+      (((uintptr_t)z | (uintptr_t)out) & run) == 0 && ((uintptr_t)weight & (w_dtype == HE_BF16 ? 7 : 15)) == 0) {
+    const int64_t units = (int64_t)rows * parts;
+    const bool wave = width <= 512;
+    // a wavefront a part, four of them a workgroup (one where there are few parts); or a workgroup a part
+    const int per = units >= 1024 ? 4 : 1;
+    const int t = wave ? 64 * per : (width <= 1024 ? 128 : width <= 4096 ? 256 : 1024);
+    const int64_t blocks = wave ? (units + per - 1) / per : units;
+    const int lanes = wave ? 64 : t;
+    const int runs = (width + 4 * lanes - 1) / (4 * lanes);
+#define GN_VEC(T, R, WAVE)                                                                                              \
+  gated_group_norm_vec_kernel<T, R, WAVE><<<(unsigned)blocks, t, 0, s>>>((T*)out, (const float*)y_f32, (const T*)z,       \
+                                                                         z_stride, weight, w_dtype, W, parts, units, eps, \
+                                                                         gate_after, out_scale)
+#define GN_RUNS(T)                                                                                                      \
+  do {                                                                                                                  \
+    if (wave && runs <= 1) GN_VEC(T, 1, true);                                                                          \
+    else if (wave) GN_VEC(T, 2, true);                                                                                  \
+    else if (runs <= 2) GN_VEC(T, 2, false);                                                                            \
+    else GN_VEC(T, 4, false);                                                                                           \
+  } while (0)
+    if (dtype == HE_BF16) GN_RUNS(bf16_t);
+    else GN_RUNS(float);
+#undef GN_RUNS
+#undef GN_VEC
+    return he_check_launch("he_gated_group_norm");
+  }
   if (dtype == HE_BF16)
     gated_group_norm_kernel<bf16_t><<<grid, threads, 0, s>>>((bf16_t*)out, (const float*)y_f32, (const bf16_t*)z, z_stride,
                                                              weight, w_dtype, W, parts, eps, gate_after, out_scale);

@@ -99,8 +99,6 @@ class DecayMemory(Mixer):
             raise RuntimeError(f"{self.prefix}: the kernel's state layout differs from the cache's")
         proj = self.qkvg(x, rows, ctx)                                   # [rows, q | k | v | g]
         y = ctx.alloc((rows, H * dv), torch.float32)
-        if ctx.padded:
-            y.zero_()           # the scan writes the rows of sequences only
         rot = self.position.rotary()
         inv_freq, half = (rot[0], rot[1] // 2) if rot is not None else (None, 0)
         floats = ops.decay_workspace_floats(rows, ctx.num_seqs, ctx.max_q_len, H, dk, dv, half)
