@@ -11,8 +11,9 @@
 // before the chunk,
 //   y_i = decay^(i+1) S^T q_i + sum over j <= i of decay^(i-j) (q_i . k_j) v_j
 //   S'  = decay^n S + sum over j of decay^(n-1-j) k_j v_j^T
-// in three launches: every chunk's own share of S' (all chunks at once), the memory before every chunk (one walk over
-// the chunks of a sequence, element by element), and every chunk's rows (all at once). A chunk begins at the first row
+// in four launches: the rows made ready (rotated, scaled, as 32-bit numbers), every chunk's own share of S' (all chunks
+// at once), the memory before every chunk (one walk over the chunks of a sequence, element by element), and every chunk's
+// rows (all at once). A chunk begins at the first row
 // a step brings, every power of the decay is at most the decay's own, and no exponent is ever positive: how the rows
 // were cut shows in rounding only. The powers come from a table [H][DM_C + 1] formed in double precision on the host.
 #include "common.h"
@@ -28,11 +29,11 @@
 
 typedef float dm_acc __attribute__((ext_vector_type(16)));
 
-static inline int dm_dvp(int dv) { return (dv + 3) / 4 * 4; }
+static inline int dm_fours(int n) { return (n + 3) / 4 * 4; }
 
 extern "C" int64_t he_decay_state_floats(int H, int dk, int dv) {
   if (H <= 0 || dk <= 0 || dv <= 0) return 0;
-  return (int64_t)H * dk * dm_dvp(dv);       // [H][dk][dv padded to 4]
+  return (int64_t)H * dk * dm_fours(dv);       // [H][dk][dv padded to 4]
 }
 
 static int64_t dm_window(int rows, int num_seqs, int64_t memory) {
@@ -42,100 +43,22 @@ static int64_t dm_window(int rows, int num_seqs, int64_t memory) {
   return chunks < most ? chunks : (most < 1 ? 1 : most);
 }
 
-extern "C" int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv, int half) {
+extern "C" int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv) {
   if (rows <= 0 || num_seqs <= 0 || max_q_len <= DM_WALK) return 0;
-  const int64_t tables = ((int64_t)rows * half + 3) / 4 * 4 * 2;
-  return tables + dm_window(rows, num_seqs, he_decay_state_floats(H, dk, dv)) * he_decay_state_floats(H, dk, dv);
+  const int64_t ready = (int64_t)rows * H * (2 * dm_fours(dk) + dm_fours(dv));
+  return ready + dm_window(rows, num_seqs, he_decay_state_floats(H, dk, dv)) * he_decay_state_floats(H, dk, dv);
 }
 
 __device__ __forceinline__ float dm_silu(float z) { return z / (1.f + expf(-z)); }
 
-// ---- loads ---------------------------------------------------------------------------------------------
 __device__ __forceinline__ void dm_vec4(float* x, const float* p) {
   const float4 v = *reinterpret_cast<const float4*>(p);
   x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
 }
-// elements d .. d + 3 of a head's `width` (zeros beyond it), one by one, through SiLU if act
-template <typename T>
-__device__ __forceinline__ void dm_load4(float* x, const T* p, int d, int width, int act) {
-#pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    x[e] = d + e < width ? to_float(p[d + e]) : 0.f;
-    if (act) x[e] = dm_silu(x[e]);
-  }
-}
-
-// The same of a query or key: rotated (cs, sn: the row's cosines and sines of the half frequencies) and scaled
-template <typename T>
-__device__ __forceinline__ void dm_load_qk4(float* x, const T* p, int d, int dk, int act, int half, const float* cs,
-                                            const float* sn, float scale) {
-  dm_load4<T>(x, p, d, dk, act);
-#pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    if (d + e < 2 * half) {
-      const bool lo = d + e < half;
-      const int i = lo ? d + e : d + e - half;
-      float y = to_float(p[lo ? d + e + half : i]);
-      if (act) y = dm_silu(y);
-      x[e] = lo ? x[e] * cs[i] - y * sn[i] : x[e] * cs[i] + y * sn[i];
-    }
-    x[e] *= scale;
-  }
-}
-
-// The whole-piece loads of a thread's share of a tile, N rows of it at dims d .. d + 3: asked for all together, with
-// no condition around them (rows past the chunk and dims past the head read the nearest ones there are and are dropped
-// afterwards), and turned into numbers when all are under way.
-template <typename T> struct DmPiece;
-template <> struct DmPiece<bf16_t> { typedef uint2 type; };
-template <> struct DmPiece<float> { typedef float4 type; };
-__device__ __forceinline__ void dm_unpack(float* x, const uint2& v) {
+__device__ __forceinline__ void dm_vec4(float* x, const bf16_t* p) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p);
   x[0] = __uint_as_float(v.x << 16); x[1] = __uint_as_float(v.x & 0xffff0000u);
   x[2] = __uint_as_float(v.y << 16); x[3] = __uint_as_float(v.y & 0xffff0000u);
-}
-__device__ __forceinline__ void dm_unpack(float* x, const float4& v) {
-  x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
-}
-
-// where dim d's partner and frequency are (a dim that is not rotated: itself, and the first frequency)
-struct DmPair {
-  int own, partner, freq;
-  bool rotated, low;
-};
-__device__ __forceinline__ DmPair dm_pair(int d, int width, int half) {
-  DmPair p;
-  p.own = d < width ? d : 0;
-  p.rotated = p.own < 2 * half;
-  p.low = p.own < half;
-  p.freq = p.rotated ? (p.low ? p.own : p.own - half) : 0;
-  p.partner = p.rotated ? (p.low ? p.own + half : p.freq) : p.own;
-  return p;
-}
-template <typename T>
-__device__ __forceinline__ typename DmPiece<T>::type dm_ask(const T* p) {
-  return *reinterpret_cast<const typename DmPiece<T>::type*>(p);
-}
-// the asked pieces as numbers: SiLU, rotation, factor; keep false: zeros
-template <typename P>
-__device__ __forceinline__ float4 dm_give(const P& own, const P& partner, const float4& c4, const float4& s4, const DmPair& p,
-                                          int act, float scale, bool keep) {
-  float x[4];
-  dm_unpack(x, own);
-  if (act) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = dm_silu(x[e]);
-  }
-  if (p.rotated) {
-    float y[4];
-    dm_unpack(y, partner);
-    const float c[4] = {c4.x, c4.y, c4.z, c4.w}, sn[4] = {s4.x, s4.y, s4.z, s4.w};
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      if (act) y[e] = dm_silu(y[e]);
-      x[e] = p.low ? x[e] * c[e] - y[e] * sn[e] : x[e] * c[e] + y[e] * sn[e];
-    }
-  }
-  return keep ? make_float4(x[0] * scale, x[1] * scale, x[2] * scale, x[3] * scale) : make_float4(0.f, 0.f, 0.f, 0.f);
 }
 
 // ---- which chunk is whose ------------------------------------------------------------------------------
@@ -167,28 +90,15 @@ __device__ __forceinline__ bool dm_find(int t, const int32_t* __restrict__ cu, i
   return false;
 }
 
-// cosines and sines of every row's position, [rows][half] each
-__global__ void dm_rotary_kernel(float* __restrict__ cs, float* __restrict__ sn, const int32_t* __restrict__ positions,
-                                 const float* __restrict__ inv_freq, int64_t n, int half) {
-  const int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x;
-  if (i >= n) return;
-  float s, c;
-  sincos_angle((float)positions[i / half] * inv_freq[i % half], &s, &c);
-  cs[i] = c;
-  sn[i] = s;
-}
-
 // what every kernel of a scan reads
 template <typename T>
 struct DmArgs {
-  const T* q;
+  const T* q;                // the projected rows
   const T* k;
   const T* v;
   int64_t stride;            // elements between rows
   const float* powers;       // [H][DM_C + 1]: decay^0 .. decay^DM_C
   const float* inv_freq;     // [half]
-  const float* cs;           // [rows][half] each, where chunks are used
-  const float* sn;
   int half;
   int act;                   // q, k and v pass SiLU
   float k_scale;
@@ -196,17 +106,76 @@ struct DmArgs {
   const int32_t* cu;
   const int32_t* slot;
   int rows;                  // of the step; those from cu[num_seqs] on belong to no sequence
-  int num_seqs, H, dk, dv, dvp;
+  int num_seqs, H, dk, dv;
+  int dkp, dvp;              // dk and dv in fours
   uint8_t* state;
   int64_t state_stride, state_offset;
-  float* ws;                 // the window's memories, [chunk of the window][H][dk][dvp]
+  // where chunks are used: the rows ready for the products, [rows][H][dkp] and [rows][H][dvp], and the window's
+  // memories, [chunk of the window][H][dk][dvp]
+  float* qf;
+  float* kf;
+  float* vf;
+  float* ws;
 };
+
+// ---- the rows made ready for the chunks' products --------------------------------------------------------
+// One workgroup a row: q, k and v as 32-bit numbers in heads of whole fours (zeros behind a head's own), through SiLU,
+// q and k rotated by the row's position, k times its factor. VEC: widths and strides in fours, so that four neighbours
+// (and their four partners in the rotation) are one load.
+#define DM_MAX_HALF (DM_MAX_KEY / 2)
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void dm_ready_kernel(DmArgs<T> a) {
+  __shared__ float cs[DM_MAX_HALF], sn[DM_MAX_HALF];
+  const int64_t row = blockIdx.x;
+  if (row >= a.cu[a.num_seqs]) return;
+  for (int i = threadIdx.x; i < a.half; i += 256) sincos_angle((float)a.positions[row] * a.inv_freq[i], sn + i, cs + i);
+  __syncthreads();
+  const int qn = a.H * a.dkp / 4, vn = a.H * a.dvp / 4;
+  for (int it = threadIdx.x; it < 2 * qn + vn; it += 256) {
+    const int part = it < qn ? 0 : it < 2 * qn ? 1 : 2;          // q, k, v
+    const int idx = it - part * qn, width = part == 2 ? a.dv : a.dk, wp = part == 2 ? a.dvp : a.dkp;
+    const int h = 4 * idx / wp, d = 4 * idx - h * wp;
+    const T* p = (part == 0 ? a.q : part == 1 ? a.k : a.v) + row * a.stride + (int64_t)h * width;
+    float* out = (part == 0 ? a.qf : part == 1 ? a.kf : a.vf) + (row * a.H + h) * wp + d;
+    float x[4], y[4] = {0.f, 0.f, 0.f, 0.f};
+    const bool turns = part < 2 && d < 2 * a.half;
+    if (VEC) {
+      dm_vec4(x, p + d);
+      if (turns) dm_vec4(y, p + (d < a.half ? d + a.half : d - a.half));
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        x[e] = d + e < width ? to_float(p[d + e]) : 0.f;
+        if (turns && d + e < 2 * a.half) y[e] = to_float(p[d + e < a.half ? d + e + a.half : d + e - a.half]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (a.act) x[e] = dm_silu(x[e]);
+      if (turns && d + e < 2 * a.half) {
+        if (a.act) y[e] = dm_silu(y[e]);
+        const bool low = d + e < a.half;
+        const int i = low ? d + e : d + e - a.half;
+        x[e] = low ? x[e] * cs[i] - y[e] * sn[i] : x[e] * cs[i] + y[e] * sn[i];
+      }
+      if (part == 1) x[e] *= a.k_scale;
+    }
+    *reinterpret_cast<float4*>(out) = make_float4(x[0], x[1], x[2], x[3]);
+  }
+}
+
+// Four numbers at dim d of a row of a chunk (n rows from `first` on, `stride` floats apart), zeros beyond the chunk or
+// the head; the load itself stands behind no condition, so that a tile's loads go out together.
+__device__ __forceinline__ float4 dm_tile4(const float* first, int64_t stride, int row, int n, int d, int width) {
+  const float4 v = *reinterpret_cast<const float4*>(first + min(row, n - 1) * stride + (d < width ? d : 0));
+  return row < n && d < width ? v : make_float4(0.f, 0.f, 0.f, 0.f);
+}
 
 // ---- every chunk's own share of the memory behind it -----------------------------------------------------
 // One workgroup of four wavefronts a (64 key dims x 64 value dims, head, chunk); a wavefront 32 x 32 of it, two rows
 // of the chunk an instruction (v_mfma_f32_32x32x2_f32: A lane l holds A[l % 32][l / 32], B likewise, D register r
 // of lane l is D[8 (r / 4) + 4 (l / 32) + r % 4][l % 32]).
-template <typename T, bool VEC>
+template <typename T>
 __global__ __launch_bounds__(256) void dm_share_kernel(DmArgs<T> a, int t0) {
   __shared__ __attribute__((aligned(16))) float ks[DM_C * DM_LD], vs[DM_C * DM_LD];
   const int h = blockIdx.y;
@@ -218,49 +187,24 @@ __global__ __launch_bounds__(256) void dm_share_kernel(DmArgs<T> a, int t0) {
   const int64_t r0 = a.cu[seq] + (int64_t)chunk * DM_C;
   const int n = min(DM_C, (int)(a.cu[seq + 1] - r0));
   const float* pw = a.powers + h * (DM_C + 1);
-  const int t = threadIdx.x;
-  if (VEC) {
-    const int d = 4 * (t & 15);
-    const DmPair kp = dm_pair(d0 + d, a.dk, a.half);
-    const int vd = c0 + d < a.dv ? c0 + d : 0;
-    typename DmPiece<T>::type kx[4], ky[4], vx[4];
-    float4 c4[4], s4[4];
-    float fade[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int row = min((t >> 4) + 16 * i, n - 1);
-      const int64_t at = (r0 + row) * a.stride, turn = (r0 + row) * a.half + kp.freq;
-      kx[i] = dm_ask(a.k + at + (int64_t)h * a.dk + kp.own);
-      if (a.half > 0) {
-        ky[i] = dm_ask(a.k + at + (int64_t)h * a.dk + kp.partner);
-        c4[i] = *reinterpret_cast<const float4*>(a.cs + turn);
-        s4[i] = *reinterpret_cast<const float4*>(a.sn + turn);
-      }
-      vx[i] = dm_ask(a.v + at + (int64_t)h * a.dv + vd);
-      fade[i] = pw[n - 1 - row];
-    }
-    const DmPair vp = dm_pair(0, 1, 0);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int row = (t >> 4) + 16 * i;
-      *reinterpret_cast<float4*>(ks + row * DM_LD + d) =
-          dm_give(kx[i], ky[i], c4[i], s4[i], kp, a.act, a.k_scale * fade[i], row < n && d0 + d < a.dk);
-      *reinterpret_cast<float4*>(vs + row * DM_LD + d) =
-          dm_give(vx[i], vx[i], c4[i], s4[i], vp, a.act, 1.f, row < n && c0 + d < a.dv);
-    }
-  } else
+  const int t = threadIdx.x, d = 4 * (t & 15);
+  const float* kr = a.kf + (r0 * a.H + h) * a.dkp;
+  const float* vr = a.vf + (r0 * a.H + h) * a.dvp;
+  float4 kx[4], vx[4];
+  float fade[4];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int row = (t >> 4) + 16 * i, d = 4 * (t & 15);
-    float kx[4] = {0.f, 0.f, 0.f, 0.f}, vx[4] = {0.f, 0.f, 0.f, 0.f};
-    if (row < n) {
-      const int64_t at = (r0 + row) * a.stride;
-      dm_load_qk4<T>(kx, a.k + at + (int64_t)h * a.dk, d0 + d, a.dk, a.act, a.half, a.cs + (r0 + row) * a.half,
-                          a.sn + (r0 + row) * a.half, a.k_scale * pw[n - 1 - row]);
-      dm_load4<T>(vx, a.v + at + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
-    }
-    *reinterpret_cast<float4*>(ks + row * DM_LD + d) = make_float4(kx[0], kx[1], kx[2], kx[3]);
-    *reinterpret_cast<float4*>(vs + row * DM_LD + d) = make_float4(vx[0], vx[1], vx[2], vx[3]);
+    const int row = (t >> 4) + 16 * i;
+    kx[i] = dm_tile4(kr, (int64_t)a.H * a.dkp, row, n, d0 + d, a.dkp);
+    vx[i] = dm_tile4(vr, (int64_t)a.H * a.dvp, row, n, c0 + d, a.dvp);
+    fade[i] = pw[max(n - 1 - row, 0)];
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int row = (t >> 4) + 16 * i;
+    *reinterpret_cast<float4*>(ks + row * DM_LD + d) =
+        make_float4(kx[i].x * fade[i], kx[i].y * fade[i], kx[i].z * fade[i], kx[i].w * fade[i]);
+    *reinterpret_cast<float4*>(vs + row * DM_LD + d) = vx[i];
   }
   __syncthreads();
   const int wave = t >> 6, l32 = t & 31, hl = (t >> 5) & 1;
@@ -277,8 +221,8 @@ __global__ __launch_bounds__(256) void dm_share_kernel(DmArgs<T> a, int t0) {
   const int col = c0 + j0 + l32;
 #pragma unroll
   for (int r = 0; r < 16; ++r) {
-    const int d = d0 + i0 + 8 * (r >> 2) + 4 * hl + (r & 3);
-    if (d < a.dk && col < a.dvp) out[(int64_t)d * a.dvp + col] = acc[r];
+    const int od = d0 + i0 + 8 * (r >> 2) + 4 * hl + (r & 3);
+    if (od < a.dk && col < a.dvp) out[(int64_t)od * a.dvp + col] = acc[r];
   }
 }
 
@@ -340,7 +284,7 @@ __global__ __launch_bounds__(256) void dm_carry_kernel(DmArgs<T> a, int t0, int 
 // window's (`tail`): the step's rows that belong to no sequence get zeros.
 #define DM_KB 32      // key dims of a block here
 #define DM_KLD 36     // floats between its rows in LDS
-template <typename T, bool VEC>
+template <typename T>
 __global__ __launch_bounds__(256, 4) void dm_rows_kernel(float* __restrict__ y, DmArgs<T> a, int t0, int tail) {
   // rows of q, rows of k, key dims of the memory; later the square and the values
   __shared__ __attribute__((aligned(16))) float lds[2 * DM_C * DM_LD];
@@ -368,6 +312,8 @@ __global__ __launch_bounds__(256, 4) void dm_rows_kernel(float* __restrict__ y, 
   const int i0 = (wave >> 1) * 32, j0 = (wave & 1) * 32;
   if (t <= DM_C) pw[t] = a.powers[h * (DM_C + 1) + t];
   const float* S = a.ws + ((int64_t)blockIdx.z * a.H + h) * a.dk * a.dvp;
+  const float* qr = a.qf + (r0 * a.H + h) * a.dkp;
+  const float* kr = a.kf + (r0 * a.H + h) * a.dkp;
   dm_acc square = {0.f}, out = {0.f};
   for (int d0 = 0; d0 < a.dk; d0 += DM_KB) {
     // thread t: rows t / 8 + 32 i and dims 4 (t % 8) of q and k; dims t / 16 + 16 i and columns 4 (t % 16) of the memory
@@ -380,44 +326,10 @@ __global__ __launch_bounds__(256, 4) void dm_rows_kernel(float* __restrict__ y, 
       const float4 v = *reinterpret_cast<const float4*>(S + (there ? (int64_t)sd * a.dvp + c0 + sc : 0));
       sx[i] = there ? v : make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    if (VEC) {
-      const DmPair p = dm_pair(d0 + d, a.dk, a.half);
-      typename DmPiece<T>::type qo[2], qp[2], ko[2], kp[2];
-      float4 c4[2], s4[2];
 #pragma unroll
-      for (int i = 0; i < 2; ++i) {
-        const int row = min((t >> 3) + 32 * i, n - 1);
-        const int64_t at = (r0 + row) * a.stride + (int64_t)h * a.dk, turn = (r0 + row) * a.half + p.freq;
-        qo[i] = dm_ask(a.q + at + p.own);
-        ko[i] = dm_ask(a.k + at + p.own);
-        if (a.half > 0) {
-          qp[i] = dm_ask(a.q + at + p.partner);
-          kp[i] = dm_ask(a.k + at + p.partner);
-          c4[i] = *reinterpret_cast<const float4*>(a.cs + turn);
-          s4[i] = *reinterpret_cast<const float4*>(a.sn + turn);
-        }
-      }
-#pragma unroll
-      for (int i = 0; i < 2; ++i) {
-        const bool keep = (t >> 3) + 32 * i < n && d0 + d < a.dk;
-        qx[i] = dm_give(qo[i], qp[i], c4[i], s4[i], p, a.act, 1.f, keep);
-        kx[i] = dm_give(ko[i], kp[i], c4[i], s4[i], p, a.act, a.k_scale, keep);
-      }
-    } else {
-#pragma unroll
-      for (int i = 0; i < 2; ++i) {
-        const int row = (t >> 3) + 32 * i;
-        float q4[4] = {0.f, 0.f, 0.f, 0.f}, k4[4] = {0.f, 0.f, 0.f, 0.f};
-        if (row < n) {
-          const int64_t at = (r0 + row) * a.stride + (int64_t)h * a.dk;
-          const float* cs = a.cs + (r0 + row) * a.half;
-          const float* sn = a.sn + (r0 + row) * a.half;
-          dm_load_qk4<T>(q4, a.q + at, d0 + d, a.dk, a.act, a.half, cs, sn, 1.f);
-          dm_load_qk4<T>(k4, a.k + at, d0 + d, a.dk, a.act, a.half, cs, sn, a.k_scale);
-        }
-        qx[i] = make_float4(q4[0], q4[1], q4[2], q4[3]);
-        kx[i] = make_float4(k4[0], k4[1], k4[2], k4[3]);
-      }
+    for (int i = 0; i < 2; ++i) {
+      qx[i] = dm_tile4(qr, (int64_t)a.H * a.dkp, (t >> 3) + 32 * i, n, d0 + d, a.dkp);
+      kx[i] = dm_tile4(kr, (int64_t)a.H * a.dkp, (t >> 3) + 32 * i, n, d0 + d, a.dkp);
     }
     __syncthreads();
 #pragma unroll
@@ -442,25 +354,9 @@ __global__ __launch_bounds__(256, 4) void dm_rows_kernel(float* __restrict__ y, 
   float4 vx[4];
   {
     const int d = 4 * (t & 15);
-    if (VEC) {
-      typename DmPiece<T>::type v[4];
-      const DmPair p = dm_pair(0, 1, 0);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        v[i] = dm_ask(a.v + (r0 + min((t >> 4) + 16 * i, n - 1)) * a.stride + (int64_t)h * a.dv + (c0 + d < a.dv ? c0 + d : 0));
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        vx[i] = dm_give(v[i], v[i], make_float4(0.f, 0.f, 0.f, 0.f), make_float4(0.f, 0.f, 0.f, 0.f), p, a.act, 1.f,
-                        (t >> 4) + 16 * i < n && c0 + d < a.dv);
-    } else {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int row = (t >> 4) + 16 * i;
-        float v4[4] = {0.f, 0.f, 0.f, 0.f};
-        if (row < n) dm_load4<T>(v4, a.v + (r0 + row) * a.stride + (int64_t)h * a.dv, c0 + d, a.dv, a.act);
-        vx[i] = make_float4(v4[0], v4[1], v4[2], v4[3]);
-      }
-    }
+    for (int i = 0; i < 4; ++i)
+      vx[i] = dm_tile4(a.vf + (r0 * a.H + h) * a.dvp, (int64_t)a.H * a.dvp, (t >> 4) + 16 * i, n, c0 + d, a.dvp);
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < 4; ++i) *reinterpret_cast<float4*>(vs + ((t >> 4) + 16 * i) * DM_LD + d) = vx[i];
@@ -592,30 +488,26 @@ static int dm_run(float* y, DmArgs<T> a, int rows, int max_q_len, float* workspa
     else dm_step_kernel<T, 16><<<grid, 256, 0, s>>>(y, a);
     return he_check_launch("he_decay_scan");
   }
-  const int64_t table = ((int64_t)rows * a.half + 3) / 4 * 4;
-  if (a.half > 0) {
-    const int64_t n = (int64_t)rows * a.half;
-    dm_rotary_kernel<<<(int)((n + 255) / 256), 256, 0, s>>>(workspace, workspace + table, a.positions, a.inv_freq, n, a.half);
-  }
-  a.cs = workspace;
-  a.sn = workspace + table;
-  a.ws = workspace + 2 * table;
+  a.qf = workspace;
+  a.kf = a.qf + (int64_t)rows * a.H * a.dkp;
+  a.vf = a.kf + (int64_t)rows * a.H * a.dkp;
+  a.ws = a.vf + (int64_t)rows * a.H * a.dvp;
   const int64_t memory = (int64_t)a.H * a.dk * a.dvp;
   const int window = (int)dm_window(rows, a.num_seqs, memory);
   const int chunks = rows / DM_C + a.num_seqs;
   const bool vec = a.dk % 4 == 0 && a.dv % 4 == 0 && a.half % 4 == 0 && a.stride % 4 == 0 &&
                    (((uintptr_t)a.q | (uintptr_t)a.k | (uintptr_t)a.v) & (4 * sizeof(T) - 1)) == 0;
+  if (vec) dm_ready_kernel<T, true><<<rows, 256, 0, s>>>(a);
+  else dm_ready_kernel<T, false><<<rows, 256, 0, s>>>(a);
   const int kb = (a.dk + DM_B - 1) / DM_B, vb = (a.dvp + DM_B - 1) / DM_B;
   for (int t0 = 0; t0 < chunks; t0 += window) {
     const int nt = chunks - t0 < window ? chunks - t0 : window;
     const dim3 share(kb * vb, a.H, nt), carry((unsigned)(((int64_t)a.dk * a.dvp / 4 + 255) / 256), a.H, a.num_seqs);
     const int tail = t0 + nt >= chunks;
     const dim3 out(vb, a.H, nt + tail);
-    if (vec) dm_share_kernel<T, true><<<share, 256, 0, s>>>(a, t0);
-    else dm_share_kernel<T, false><<<share, 256, 0, s>>>(a, t0);
+    dm_share_kernel<T><<<share, 256, 0, s>>>(a, t0);
     dm_carry_kernel<T><<<carry, 256, 0, s>>>(a, t0, nt);
-    if (vec) dm_rows_kernel<T, true><<<out, 256, 0, s>>>(y, a, t0, tail);
-    else dm_rows_kernel<T, false><<<out, 256, 0, s>>>(y, a, t0, tail);
+    dm_rows_kernel<T><<<out, 256, 0, s>>>(y, a, t0, tail);
   }
   return he_check_launch("he_decay_scan");
 }
@@ -634,17 +526,17 @@ extern "C" int he_decay_scan(void* y_f32, const void* q, const void* k, const vo
   HE_REQUIRE(state != nullptr && state_offset % 16 == 0 && state_stride % 16 == 0 && ((uintptr_t)state & 15) == 0 &&
                  state_stride >= state_offset + 4 * he_decay_state_floats(H, dk, dv),
              "he_decay_scan: the state row is too short or not aligned");
-  const int64_t need = he_decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv, half);
+  const int64_t need = he_decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv);
   HE_REQUIRE(need == 0 || (workspace_f32 != nullptr && workspace_floats >= need && ((uintptr_t)workspace_f32 & 15) == 0),
              "he_decay_scan: the workspace has %lld floats of %lld, or is not aligned", (long long)workspace_floats, (long long)need);
   if (rows == 0 || num_seqs == 0) return 0;
 #define DM_FILL(T)                                                                                                     \
   DmArgs<T> a;                                                                                                         \
   a.q = (const T*)q; a.k = (const T*)k; a.v = (const T*)v; a.stride = in_stride; a.powers = (const float*)powers_f32;   \
-  a.inv_freq = (const float*)inv_freq_f32; a.cs = a.sn = nullptr; a.half = half; a.act = act; a.k_scale = k_scale;     \
+  a.inv_freq = (const float*)inv_freq_f32; a.half = half; a.act = act; a.k_scale = k_scale;     \
   a.positions = (const int32_t*)positions; a.cu = (const int32_t*)cu_seqlens; a.slot = (const int32_t*)seq_slot;       \
-  a.rows = rows; a.num_seqs = num_seqs; a.H = H; a.dk = dk; a.dv = dv; a.dvp = dm_dvp(dv); a.state = (uint8_t*)state;                 \
-  a.state_stride = state_stride; a.state_offset = state_offset; a.ws = nullptr;                                        \
+  a.rows = rows; a.num_seqs = num_seqs; a.H = H; a.dk = dk; a.dv = dv; a.dkp = dm_fours(dk); a.dvp = dm_fours(dv); a.state = (uint8_t*)state;                 \
+  a.state_stride = state_stride; a.state_offset = state_offset; a.qf = a.kf = a.vf = a.ws = nullptr;                   \
   return dm_run<T>((float*)y_f32, a, rows, max_q_len, (float*)workspace_f32, (hipStream_t)stream)
   if (dtype == HE_BF16) {
     DM_FILL(bf16_t);

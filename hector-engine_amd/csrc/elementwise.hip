@@ -63,8 +63,22 @@ __global__ __launch_bounds__(1024) void embedding_normed_kernel(float* __restric
 #pragma unroll
   for (int u = 0; u < 2; ++u) {        // the gains are on their way before the row's sum is formed
     const int i = 8 * (threadIdx.x + u * blockDim.x);
+    const int at = i < D ? i : 0;
+    if (w_dtype == HE_BF16) {
+      const uint4 v = *reinterpret_cast<const uint4*>((const uint16_t*)norm_w + at);
+      const uint32_t w[4] = {v.x, v.y, v.z, v.w};
 #pragma unroll
-    for (int j = 0; j < 8; ++j) g[8 * u + j] = load_param(norm_w, (i < D ? i : 0) + j, w_dtype);
+      for (int j = 0; j < 4; ++j) {
+        g[8 * u + 2 * j] = __uint_as_float(w[j] << 16);
+        g[8 * u + 2 * j + 1] = __uint_as_float(w[j] & 0xffff0000u);
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; j += 4) {
+        const float4 v = *reinterpret_cast<const float4*>((const float*)norm_w + at + j);
+        g[8 * u + j] = v.x; g[8 * u + j + 1] = v.y; g[8 * u + j + 2] = v.z; g[8 * u + j + 3] = v.w;
+      }
+    }
   }
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
@@ -101,7 +115,7 @@ extern "C" int he_embedding(void* out_f32, const void* table, const void* ids, i
   hipStream_t s = (hipStream_t)stream;
   HE_REQUIRE(norm_w == nullptr || w_dtype == HE_F32 || w_dtype == HE_BF16, "he_embedding: bad weight dtype");
   if (norm_w != nullptr && table_dtype == HE_BF16 && D % 8 == 0 && D <= 16 * 1024 &&
-      (((uintptr_t)table | (uintptr_t)out_f32) & 15) == 0) {
+      (((uintptr_t)table | (uintptr_t)out_f32 | (uintptr_t)norm_w) & 15) == 0) {
     int wide = 64;
     while (wide < 256 ? 8 * wide < D : 16 * wide < D) wide <<= 1;
     embedding_normed_kernel<<<rows, wide, 0, s>>>((float*)out_f32, (const uint16_t*)table, (const int32_t*)ids, D, V, scale,

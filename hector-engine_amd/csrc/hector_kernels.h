@@ -362,7 +362,7 @@ int he_delta_scan(void* y_f32, const void* q, const void* k, const void* v, int6
 // sequence's row of the state area, zeros at a sequence's start, and is carried on. max_q_len: the most rows of a
 // sequence in this step. Rows of y that belong to no sequence get zeros. workspace_f32: he_decay_workspace_floats floats on a 16-byte boundary. dk up to 512.
 int64_t he_decay_state_floats(int H, int dk, int dv);
-int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv, int half);
+int64_t he_decay_workspace_floats(int rows, int num_seqs, int max_q_len, int H, int dk, int dv);
 int he_decay_scan(void* y_f32, const void* q, const void* k, const void* v, int64_t in_stride, const void* powers_f32,
                   int act, float k_scale, const void* inv_freq_f32, int half, const void* positions, void* state,
                   int64_t state_stride, int64_t state_offset, const void* cu_seqlens, const void* seq_slot, int rows,

@@ -79,7 +79,7 @@ _SIGNATURES = {
     "he_route_tokens": [c_ptr, c_ptr, c_ptr, c_ptr, c_ptr, c_int, c_ptr, c_int, c_ptr, c_int, c_int, c_int, c_int,
                         c_int, c_int, c_int, c_f32, c_int, c_ptr, c_int, c_int, c_ptr],
     "he_decay_state_floats": [c_int, c_int, c_int],
-    "he_decay_workspace_floats": [c_int, c_int, c_int, c_int, c_int, c_int, c_int],
+    "he_decay_workspace_floats": [c_int, c_int, c_int, c_int, c_int, c_int],
     "he_decay_scan": [c_ptr, c_ptr, c_ptr, c_ptr, c_i64, c_ptr, c_int, c_f32, c_ptr, c_int, c_ptr, c_ptr, c_i64, c_i64, c_ptr,
                       c_ptr, c_int, c_int, c_int, c_int, c_int, c_int, c_ptr, c_i64, c_int, c_ptr],
     "he_delta_state_floats": [c_int, c_int, c_int],

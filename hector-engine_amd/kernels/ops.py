@@ -686,9 +686,9 @@ def decay_state_floats(H: int, dk: int, dv: int) -> int:
     return int(_lib.load().he_decay_state_floats(H, dk, dv))
 
 
-def decay_workspace_floats(rows: int, num_seqs: int, max_q_len: int, H: int, dk: int, dv: int, half: int) -> int:
+def decay_workspace_floats(rows: int, num_seqs: int, max_q_len: int, H: int, dk: int, dv: int) -> int:
     """Floats of workspace decay_scan wants for a step of these sizes (0: none)."""
-    return int(_lib.load().he_decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv, half))
+    return int(_lib.load().he_decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv))
 
 
 @_op("decay_scan")
@@ -721,7 +721,7 @@ def decay_scan(y, q, k, v, powers, state, state_offset: int, positions, cu_seqle
         _need(t, name, torch.int32)
         if t.numel() < n:
             raise ValueError(f"decay_scan: {name} shorter than the step")
-    need = decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv, half)
+    need = decay_workspace_floats(rows, num_seqs, max_q_len, H, dk, dv)
     if workspace is None and need:
         workspace = torch.empty(need, dtype=torch.float32, device=y.device)
     if workspace is not None:

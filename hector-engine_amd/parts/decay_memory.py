@@ -100,8 +100,8 @@ class DecayMemory(Mixer):
         proj = self.qkvg(x, rows, ctx)                                   # [rows, q | k | v | g]
         y = ctx.alloc((rows, H * dv), torch.float32)
         rot = self.position.rotary()
-        inv_freq, half = (rot[0], rot[1] // 2) if rot is not None else (None, 0)
-        floats = ops.decay_workspace_floats(rows, ctx.num_seqs, ctx.max_q_len, H, dk, dv, half)
+        inv_freq = rot[0] if rot is not None else None
+        floats = ops.decay_workspace_floats(rows, ctx.num_seqs, ctx.max_q_len, H, dk, dv)
         ws = ctx.alloc((floats,), torch.float32) if floats else None
         ops.decay_scan(y, proj[:, :H * dk], proj[:, H * dk:2 * H * dk], proj[:, 2 * H * dk:2 * H * dk + H * dv], self.powers,
                        cache.state, 0, ctx.positions, ctx.cu_seqlens, ctx.seq_slot, rows, ctx.num_seqs, ctx.max_q_len, H, dk,

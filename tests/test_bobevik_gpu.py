@@ -210,7 +210,7 @@ def test_memories_too_large_to_hold_for_all_chunks_at_once(ops):
     cu, slots = [0, 10, 300, T], [2, 0, 1]
     positions = [t for a, b in zip(cu, cu[1:]) for t in range(b - a)]
     state = torch.zeros(3, 4 * ops.decay_state_floats(H, dk, dv), dtype=torch.uint8, device="cuda")
-    assert ops.decay_workspace_floats(T, 3, 350, H, dk, dv, 0) < 10 * ops.decay_state_floats(H, dk, dv)     # not all 12 at once
+    assert ops.decay_workspace_floats(T, 3, 350, H, dk, dv) < 10 * ops.decay_state_floats(H, dk, dv)     # not all 12 at once
     y = scan(ops, x, state, 0, positions, cu, slots, H, dk, dv, decay, 0, 1.0, False, 0.05)
     for h in (0, 17, 39):
         one = torch.cat([x[:, (p * H + h) * dk:(p * H + h + 1) * dk] for p in range(3)], 1).contiguous()
