@@ -183,9 +183,11 @@ __device__ __forceinline__ void pw_values(floatx16 (&o)[Pw<NT>::DT], const uint4
   }
 }
 
-// ATTN_SHAPED: raw score i of a step from key_base on through the cap and the table (base-2 domain).
-template <int NT>
+// ATTN_SHAPED: raw score i of a step from key_base on through the cap and the table (base-2 domain). ATTN_CAPPED: through
+// the cap alone.
+template <int NT, int MODE>
 __device__ __forceinline__ float pw_shaped(const WideTile<NT>& t, float s, int i, int key_base, int g) {
+  if (MODE == ATTN_CAPPED) return __builtin_fmaf(-t.sh.c1, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * t.sh.k1)), t.sh.c0);
   return attn_cap(t.sh, s) + t.sh.table[min(max(t.hi - key_base - pw_key_of(i, g), 0), t.sh.last)];
 }
 
@@ -201,7 +203,7 @@ __device__ __forceinline__ bool pw_softmax(WideTile<NT>& t, const floatx16& s, i
 #pragma unroll
   for (int i = 0; i < 16; ++i) {
     const int key = key_base + pw_key_of(i, g);
-    const float x = MODE == ATTN_SHAPED ? pw_shaped<NT>(t, s[i], i, key_base, g) : s[i];
+    const float x = MODE >= ATTN_SHAPED ? pw_shaped<NT, MODE>(t, s[i], i, key_base, g) : s[i];
     v[i] = (key >= t.lo && key <= t.hi) ? x : -INFINITY;
     mx = fmaxf(mx, v[i]);
   }
@@ -303,7 +305,7 @@ __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, 
   // each, four that round two pairs and add them up; product n of P gets the pieces
   // ceil(16 n / P) .. ceil(16 (n + 1) / P) - 1. Where the scores are shaped, 16 pieces of one score each come first.
   constexpr int P = NT + 2 * DT;
-  constexpr int PIECES = MODE == ATTN_SHAPED ? 32 : 16;
+  constexpr int PIECES = MODE >= ATTN_SHAPED ? 32 : 16;
   floatx16 s_next = pw_score_start<MODE>(t.bias, t.hi, next_key_base, g);   // the scores of the step at next_key_base
   float mx = -INFINITY, m_new = t.m, sum = 0.f;
   bool moved = false;
@@ -321,7 +323,7 @@ __device__ __forceinline__ void pw_fast_step(WideTile<NT>& t, floatx16& s_pend, 
     for (int turn = (PIECES * n + P - 1) / P; turn < (PIECES * (n + 1) + P - 1) / P; ++turn) {
       const int piece = turn - (PIECES - 16);
       if (piece < 0) {
-        s_pend[turn] = pw_shaped<NT>(t, s_pend[turn], turn, next_key_base - 32, g);
+        s_pend[turn] = pw_shaped<NT, MODE>(t, s_pend[turn], turn, next_key_base - 32, g);
       } else if (piece < 4) {
 #pragma unroll
         for (int i = 4 * piece; i < 4 * piece + 4; ++i) mx = fmaxf(mx, s_pend[i]);
@@ -416,7 +418,7 @@ attention_prefill_wide_kernel(
   const int64_t k_stride = (int64_t)KVH * he_k_page_elems(HD), v_stride = (int64_t)KVH * he_v_page_elems(HD);
   const uint16_t* kp = kpool + (int64_t)kvh * he_k_page_elems(HD);
   const uint16_t* vp = vpool + (int64_t)kvh * he_v_page_elems(HD);
-  const float scale_log2 = MODE == ATTN_SHAPED ? 1.f : scale * PW_LOG2E;
+  const float scale_log2 = MODE >= ATTN_SHAPED ? 1.f : scale * PW_LOG2E;
 
   // the workgroup's pages: from the first key its first query sees to its last query
   const int blk_last = start + min(q0 + PW_QUERIES, q_len) - 1;
@@ -448,6 +450,7 @@ attention_prefill_wide_kernel(
   t.m = -INFINITY;
   t.l = 0.f;
   t.bias = MODE == ATTN_SLOPES ? ex.slopes[h] / scale : 0.f;
+  if (MODE == ATTN_CAPPED) t.sh = attn_shape_of(ex, h, scale);
   if (MODE == ATTN_SHAPED) {
     t.sh = attn_shape_of(ex, h, scale);
     const int entries = t.sh.table != nullptr ? ex.table_len : 1;
@@ -590,10 +593,12 @@ int he_attention_prefill_wide(void* out, const void* q, const void* kpool, const
       attention_prefill_wide_kernel<NTV, ATTN_SLOPES><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
     else if (mode == ATTN_SHAPED)                                                               \
       attention_prefill_wide_kernel<NTV, ATTN_SHAPED><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
+    else if (mode == ATTN_CAPPED)                                                               \
+      attention_prefill_wide_kernel<NTV, ATTN_CAPPED><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
     else                                                                                        \
       attention_prefill_wide_kernel<NTV, ATTN_RAW><<<grid, 64 * PW_WAVES, 0, s>>>(PREFILL_WIDE_ARGS); \
     break;
-  const int mode = attn_mode(ex);
+  const int mode = attn_mode(ex) == ATTN_SHAPED && ex.table == nullptr ? ATTN_CAPPED : attn_mode(ex);
   switch (hd / 16) {
     PREFILL_WIDE(1) PREFILL_WIDE(2) PREFILL_WIDE(3) PREFILL_WIDE(4)
     PREFILL_WIDE(5) PREFILL_WIDE(6) PREFILL_WIDE(7) PREFILL_WIDE(8)

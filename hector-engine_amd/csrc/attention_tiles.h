@@ -40,7 +40,8 @@ __device__ __forceinline__ bf16x8 ld8(const uint16_t* p, bool ok) {
 
 // What the scores of a kernel pass through (the kernels' template parameter MODE): nothing, a slope over the distance
 // added to the raw score, or a cap and a table over the distance (AttnShape).
-enum { ATTN_RAW = 0, ATTN_SLOPES = 1, ATTN_SHAPED = 2 };
+// ATTN_CAPPED is a cap alone, for the kernel that has a form without the table (attn_mode does not give it).
+enum { ATTN_RAW = 0, ATTN_SLOPES = 1, ATTN_SHAPED = 2, ATTN_CAPPED = 3 };
 __host__ __device__ __forceinline__ int attn_mode(const AttnExtras& ex) {
   return ex.slopes != nullptr ? ATTN_SLOPES : (ex.table != nullptr || ex.cap > 0.f) ? ATTN_SHAPED : ATTN_RAW;
 }
