@@ -1,5 +1,5 @@
 """Generation library for one MI355X (package folder ``hector-engine_amd``): Qwen2 dense decoders and
-the Volonex design, both assembled from the same registered parts.
+the other registered designs, all assembled from the same parts.
 
 Python entry point:
 

@@ -90,7 +90,7 @@ def scan(ops, x, state, offset, positions, cu, slots, H, dk, dv, decay, r, base,
     return y
 
 
-SIZES = [(2, 64, 32, 64, False), (3, 12, 20, 8, False), (1, 5, 3, 2, False), (2, 130, 24, 0, True), (4, 16, 1, 0, True), (1, 1, 7, 0, True),
+SIZES = [(2, 64, 40, 64, False), (3, 12, 20, 8, False), (1, 5, 3, 2, False), (2, 130, 24, 0, True), (4, 16, 1, 0, True), (1, 1, 7, 0, True),
          (2, 48, 66, 48, False), (1, 300, 132, 300, False), (2, 128, 256, 128, False)]
 
 
@@ -391,7 +391,7 @@ MODELS = {
     "C1": model([layer("parallel", pair(attn(4, 2, 32, 16, 0.3, rot(500.0, 16, 3.0), 8.0), memory((0.9, 0.5, 0.995), 12, 20)), 72),
                  layer("attention", attn(3, 3, 16, 24, 0.5, rot(1000.0, 8)), 40),
                  layer("attention", attn(6, 2, 16, 8, 0.4, rot(10000.0, 16), v_mix=True)),
-                 layer("retention", memory((0.97, 0.999), 24, 8, rot(10000.0, 16)), 48),
+                 layer("retention", memory((0.97, 0.9985), 24, 8, rot(10000.0, 16)), 48),
                  layer("attention", attn(4, 2, 48, 8, 0.3, rot(10000.0, 48), v_mix=True), 56)],
                 vocab=97, width=48, mult=0.6),
     "C2": model([layer("retention", memory((0.9,), 10, 6)), layer("attention", attn(1, 1, 10, 7, 0.6, v_mix=True), 30),
@@ -399,7 +399,7 @@ MODELS = {
                  layer("attention", attn(5, 1, 14, 7, 0.5, rot(100.0, 6), v_mix=True), 18)],
                 vocab=131, width=36, mult=1.3, eps=1e-4),
     "C3": model([layer("attention", attn(4, 4, 32, 32, 0.3, rot(10000.0, 32), v_mix=True), 64),
-                 layer("retention", memory((0.96875, 0.995, 0.6), 72, 136, rot(10000.0, 72)), 64),
+                 layer("retention", memory((0.95, 0.995, 0.6), 72, 136, rot(10000.0, 72)), 64),
                  layer("parallel", pair(attn(2, 1, 64, 64, 0.2, rot(10000.0, 64, 2.0), 4.0), memory((0.7, 0.99), 68, 80)), 64)],
                 vocab=64, width=64, mult=1.0),
 }
@@ -866,7 +866,7 @@ def random_configuration(rng):
             mixer = attn(kv * rng.choice([1, 2, 3]), kv, dim, e, rng.choice([0.2, 0.4]), rotation(dim, False), v_mix=mixes)
         else:
             H = rng.choice([1, 2, 3, 5])
-            mixer = memory([rng.choice([0.5, 0.9, 0.99, 0.999, 1.0 - 2.0 ** -11]) for _ in range(H)],
+            mixer = memory([rng.choice([0.5, 0.9, 0.99, 0.998, 1.0 - 2.0 ** -10]) for _ in range(H)],
                            rng.choice([4, 5, 12, 16, 40, 66, 72]), rng.choice([1, 4, 6, 16, 36, 68]))
             if kind == "retention":
                 r = rotation(mixer["dim"], False)
